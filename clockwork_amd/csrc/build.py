@@ -59,7 +59,8 @@ FLAGS = [
 PLAIN_SOURCES = {"core": "core.hip", "gemm": "gemm.hip", "gemm_tile": "gemm_tile.hip", "sampling": "sampling.hip",
                  "rowwise": "rowwise.hip", "sink_attention": "sink_attention.hip",
                  "linear_recurrence": "linear_recurrence.hip", "rows_attention": "rows_attention.hip", "moe": "moe.hip",
-                 "state_space": "state_space.hip"}
+                 "state_space": "state_space.hip", "short_conv": "short_conv.hip", "selective_scan": "selective_scan.hip",
+                 "matrix_memory": "matrix_memory.hip"}
 ATTENTION_SOURCE = "attention.hip"
 # head sizes compiled by build_all: the tests' models, the kernel tests and the benchmark's
 DEFAULT_HEAD_DIMS = (16, 32, 48, 64, 96, 128, 160, 224, 256)

@@ -63,11 +63,44 @@ __device__ __forceinline__ float cw_clipped_glu(float gate, float up, float limi
   const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
   return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
 }
+// What the kernels of gate/up products make of a gate and an up value: ``act`` > 0 the clipped gated
+// activation of that limit, < 0 max(gate, 0) * up, else silu(gate) * up.
+__device__ __forceinline__ float cw_gated(float g, float u, float act) {
+  return act > 0.0f ? cw_clipped_glu(g, u, act) : act < 0.0f ? fmaxf(g, 0.0f) * u : g / (1.0f + expf(-g)) * u;
+}
 // The tanh form of GELU, 0.5 z (1 + tanh(y)) with y = sqrt(2 / pi) (z + 0.044715 z^3), through
 // 0.5 (1 + tanh(y)) = 1 / (1 + exp(-2 y)).
 __device__ __forceinline__ float cw_gelu_tanh(float z) {
   return z / (1.0f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
 }
+
+__device__ __forceinline__ float cw_silu(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float cw_logistic(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float cw_softplus(float z) { return z > 0.0f ? z + log1pf(expf(-z)) : log1pf(expf(z)); }
+
+template <typename T, int V> struct CwVec;   // V neighbouring elements as float32
+template <typename T> struct CwVec<T, 1> {
+  static __device__ __forceinline__ void load(const T* p, float (&o)[1]) { o[0] = cw_to_float(p[0]); }
+  static __device__ __forceinline__ void store(T* p, const float (&v)[1]) { p[0] = cw_from_float<T>(v[0]); }
+};
+template <> struct CwVec<float, 4> {
+  static __device__ __forceinline__ void load(const float* p, float (&o)[4]) {
+    const float4 v = *reinterpret_cast<const float4*>(p);
+    o[0] = v.x; o[1] = v.y; o[2] = v.z; o[3] = v.w;
+  }
+  static __device__ __forceinline__ void store(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+};
+template <> struct CwVec<bf16_t, 4> {
+  static __device__ __forceinline__ void load(const bf16_t* p, float (&o)[4]) {
+    const uint2 d = *reinterpret_cast<const uint2*>(p);
+    o[0] = __uint_as_float(d.x << 16); o[1] = __uint_as_float(d.x & 0xffff0000u);
+    o[2] = __uint_as_float(d.y << 16); o[3] = __uint_as_float(d.y & 0xffff0000u);
+  }
+  static __device__ __forceinline__ void store(bf16_t* p, const float (&v)[4]) {
+    *reinterpret_cast<uint2*>(p) = make_uint2((uint32_t)cw_float_to_bf16_bits(v[0]) | ((uint32_t)cw_float_to_bf16_bits(v[1]) << 16),
+                                              (uint32_t)cw_float_to_bf16_bits(v[2]) | ((uint32_t)cw_float_to_bf16_bits(v[3]) << 16));
+  }
+};
 
 __device__ __forceinline__ float cw_wave_sum(float v) {
 #pragma unroll

@@ -458,7 +458,7 @@ __global__ void silu_mul_kernel(const T* __restrict__ gate_up, T* __restrict__ o
     const int i = (int)(idx - t * I);
     const float g = cw_to_float(gate_up[t * 2 * I + i]);
     const float u = cw_to_float(gate_up[t * 2 * I + I + i]);
-    out[idx] = cw_from_float<T>(limit > 0.0f ? cw_clipped_glu(g, u, limit) : g / (1.0f + expf(-g)) * u);
+    out[idx] = cw_from_float<T>(cw_gated(g, u, limit));
   }
 }
 
@@ -497,14 +497,14 @@ __global__ void silu_mul_vec_kernel(const T* __restrict__ gate_up, T* __restrict
     Vec16B<T>::load(gate_up + t * 2 * I + i, g);
     Vec16B<T>::load(gate_up + t * 2 * I + I + i, u);
 #pragma unroll
-    for (int e = 0; e < N; ++e) r[e] = limit > 0.0f ? cw_clipped_glu(g[e], u[e], limit) : g[e] / (1.0f + expf(-g[e])) * u[e];
+    for (int e = 0; e < N; ++e) r[e] = cw_gated(g[e], u[e], limit);
     Vec16B<T>::store(out + t * I + i, r);
   }
 }
 
-// limit > 0: the clipped gated activation with that limit instead of silu(gate) * up
+// limit > 0: the clipped gated activation with that limit instead of silu(gate) * up; < 0: max(gate, 0) * up
 CW_EXPORT int cw_silu_mul(const void* gate_up, void* out, int dtype, int T, int I, float limit, hipStream_t stream) {
-  if (T < 0 || I <= 0 || !(limit >= 0.0f)) return CW_ERR_ARG;
+  if (T < 0 || I <= 0 || limit != limit) return CW_ERR_ARG;
   if (T == 0) return CW_OK;
   const int vec_n = dtype == CW_BF16 ? 8 : 4;
   const bool vec = (I % vec_n == 0) && !((uintptr_t)gate_up & 15) && !((uintptr_t)out & 15);

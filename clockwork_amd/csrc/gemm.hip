@@ -200,7 +200,7 @@ CW_EXPORT int cw_gemm_f32(const float* A, int64_t lda, const float* W, const flo
 // MODE 0: y bfloat16 [M, N]; MODE 4: the same with the erf GELU (``act`` > 0: its tanh form) applied
 // to the float32 sums before they are rounded; MODE 5: with max(z, 0)^2 applied to them; MODE 1: y float32 [M, N] (logits); MODE 2: W is [2I, K] with gate
 // rows first, y[m, i] = silu(gate_i) * up_i as bfloat16 [M, I] (``act`` > 0: the clipped gated
-// activation with that limit instead): a row tile holds 8 gate rows and the 8 up rows that belong to them. MODE 3: K is also split over gridDim.y workgroups, each
+// activation with that limit instead; < 0: max(gate, 0) * up): a row tile holds 8 gate rows and the 8 up rows that belong to them. MODE 3: K is also split over gridDim.y workgroups, each
 // writing its float32 partial product [split, M, N]; whoever reads y next sums the partials in
 // order (the residual-add + norm kernel does): a narrow output with a long K (96 row tiles for
 // 27 MB of weights) then streams on all compute units instead of 96.
@@ -339,7 +339,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_bf16_kernel(const bf16
       if (m >= M || i >= I) continue;
       const float g = red[0][(rt * MT + mt) * 256 + j * 16 + tok];
       const float u = red[0][(rt * MT + mt) * 256 + (j + 8) * 16 + tok];
-      ((bf16_t*)C)[(int64_t)m * ldc + i] = __float2bfloat16(act > 0.0f ? cw_clipped_glu(g, u, act) : g / (1.0f + __expf(-g)) * u);
+      ((bf16_t*)C)[(int64_t)m * ldc + i] = __float2bfloat16(act > 0.0f ? cw_clipped_glu(g, u, act) : act < 0.0f ? fmaxf(g, 0.0f) * u : g / (1.0f + __expf(-g)) * u);
     }
   } else {
     for (int idx = threadIdx.x; idx < RT * MT * 256; idx += WAVES * 64) {
@@ -507,7 +507,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_stream_bf16_kernel(const bf16
         }
         const int64_t i = (int64_t)tile * 8 + j;
         if (m < M && i < I) ((bf16_t*)C)[(int64_t)m * ldc + i] =
-              __float2bfloat16(act > 0.0f ? cw_clipped_glu(g, up, act) : g / (1.0f + __expf(-g)) * up);
+              __float2bfloat16(act > 0.0f ? cw_clipped_glu(g, up, act) : act < 0.0f ? fmaxf(g, 0.0f) * up : g / (1.0f + __expf(-g)) * up);
       }
     } else {
       for (int idx = threadIdx.x; idx < MT * 256; idx += WAVES * 64) {  // (token, j): 16 outputs side by side
@@ -799,13 +799,13 @@ CW_EXPORT int cw_gemm_bf16_swiglu_normed(const float* resid, const void* delta, 
 
 // y = x W^T for M <= 64 rows of bfloat16 x [M, K] (row stride ldx) and bfloat16 W [N, K].
 // mode 0: y bfloat16 [M, N] (4: gelu(y), the erf form, with ``act`` > 0 the tanh form; 5: max(y, 0)^2);
-// 1: y float32 [M, N]; 2: y = silu(gate) * up, with ``act`` > 0 the clipped gated activation of that limit, bfloat16 [M, N / 2];
+// 1: y float32 [M, N]; 2: y = silu(gate) * up, with ``act`` > 0 the clipped gated activation of that limit, < 0 max(gate, 0) * up, bfloat16 [M, N / 2];
 // 3: float32 partial products [splits, M, N], splits = ``k_splits`` if that is positive (up to 16
 // rows of x; what a caller has measured to be the best for the shape), else
 // cw_gemm_bf16_skinny_ksplits(M, N, K). K must be a multiple of 8 (16-byte rows).
 CW_EXPORT int cw_gemm_bf16_skinny(int mode, const void* X, int64_t ldx, const void* W, void* C,
                                   int64_t ldc, int M, int N, int K, int k_splits, float act, hipStream_t stream) {
-  if (M < 0 || N <= 0 || K <= 0 || mode < 0 || mode > 5 || !(act >= 0.0f)) return CW_ERR_ARG;
+  if (M < 0 || N <= 0 || K <= 0 || mode < 0 || mode > 5 || !(act >= 0.0f || mode == 2)) return CW_ERR_ARG;
   if (M > CW_SKINNY_MAX_M) return CW_ERR_SIZE;
   if ((K & 7) || (ldx & 7) || ((uintptr_t)X & 15) || ((uintptr_t)W & 15)) return CW_ERR_ARG;
   if (mode == 2 && (N & 1)) return CW_ERR_ARG;

@@ -48,7 +48,7 @@ struct TileArgs {
   void* C;
   int64_t ldc;
   int M, N, K;
-  float act;          // MODE 2: > 0: the clipped gated activation with this limit
+  float act;          // MODE 2: > 0: the clipped gated activation with this limit, < 0: max(gate, 0) * up
 };
 
 // Row of W that row ``rb`` (0..127) of the workgroup's W tile ``tn`` is. MODE 2: a wave's 64 tile
@@ -163,7 +163,7 @@ __global__ __launch_bounds__(256, 2) void gemm_tile_bf16_kernel(TileArgs a) {
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           const float g = acc[mi][ni][e], up = acc[mi][ni + 2][e];
-          o[e] = cw_float_to_bf16_bits(a.act > 0.0f ? cw_clipped_glu(g, up, a.act) : g / (1.0f + __expf(-g)) * up);
+          o[e] = cw_float_to_bf16_bits(a.act > 0.0f ? cw_clipped_glu(g, up, a.act) : a.act < 0.0f ? fmaxf(g, 0.0f) * up : g / (1.0f + __expf(-g)) * up);
         }
         bf16_t* dst = (bf16_t*)a.C + m * a.ldc + i0;
         if (i0 + 4 <= I && !(a.ldc & 3)) {
@@ -230,7 +230,7 @@ static int gt_launch(const TileArgs& a, hipStream_t stream) {
 // mode 2: y = silu(gate) * up, bfloat16 [M, N / 2], W = [gate; up], no bias.
 CW_EXPORT int cw_gemm_bf16_tiled(int mode, const void* X, int64_t ldx, const void* W, const void* bias,
                                  int bias_f32, void* C, int64_t ldc, int M, int N, int K, float act, hipStream_t stream) {
-  if (M < 0 || N <= 0 || K <= 0 || (mode != 0 && mode != 2) || !(act >= 0.0f)) return CW_ERR_ARG;
+  if (M < 0 || N <= 0 || K <= 0 || (mode != 0 && mode != 2) || !(act >= 0.0f || mode == 2)) return CW_ERR_ARG;
   if ((K & 7) || (ldx & 7) || ldx < K || ((uintptr_t)X & 15) || ((uintptr_t)W & 15) || ((uintptr_t)C & 7))
     return CW_ERR_ARG;
   if (mode == 2 && ((N & 1) || bias != nullptr)) return CW_ERR_ARG;
@@ -274,7 +274,7 @@ CW_EXPORT int cw_gemm_bf16_tiled(int mode, const void* X, int64_t ldx, const voi
 // change places between lane rows (v_permlane16_swap) so that it stores 16 bytes and four lanes
 // 64 bytes of a row.
 //
-// MODE as above (2 with ``act`` > 0: the clipped gated activation of that limit), and 5: MODE 0 with
+// MODE as above (2 with ``act`` > 0: the clipped gated activation of that limit, < 0: max(gate, 0) * up), and 5: MODE 0 with
 // max(y, 0)^2, with ``act`` > 0 the tanh form of GELU, applied to the float32 sums (after the bias);
 // K a multiple of 64, at least 256; both matrices below 4 GiB. MODE 3: the product
 // of a narrow output with a long K (too few tiles to fill the card) summed in k_splits runs of K,
@@ -517,6 +517,8 @@ __global__ __launch_bounds__(256) void gemm_wide_bf16_kernel(WideArgs a) {
           if (a.act > 0.0f) {
             const float gl = fminf(g, a.act), ul = fminf(fmaxf(up, -a.act), a.act);
             v[e] = gl * __builtin_amdgcn_rcpf(1.0f + __expf(-1.702f * gl)) * (ul + 1.0f);
+          } else if (a.act < 0.0f) {
+            v[e] = fmaxf(g, 0.0f) * up;
           } else {
             v[e] = g * __builtin_amdgcn_rcpf(1.0f + __expf(-g)) * up;
           }
@@ -665,7 +667,7 @@ static int w_launch(WideArgs a, int workgroups, hipStream_t stream) {
 // units of the GPU (one workgroup fills a unit).
 CW_EXPORT int cw_gemm_bf16_wide(int mode, const void* X, int64_t ldx, const void* W, const void* bias, int bias_f32,
                                 void* C, int64_t ldc, int M, int N, int K, float act, int workgroups, hipStream_t stream) {
-  if (M < 0 || N <= 0 || K <= 0 || (mode != 0 && mode != 2 && mode != 5) || workgroups < 8 || !(act >= 0.0f)) return CW_ERR_ARG;
+  if (M < 0 || N <= 0 || K <= 0 || (mode != 0 && mode != 2 && mode != 5) || workgroups < 8 || !(act >= 0.0f || mode == 2)) return CW_ERR_ARG;
   if (((uintptr_t)X & 15) || ((uintptr_t)W & 15) || ((uintptr_t)C & 7)) return CW_ERR_ARG;
   if (mode == 2 && ((N & 1) || bias != nullptr)) return CW_ERR_ARG;
   if (ldc < (mode == 2 ? N / 2 : N)) return CW_ERR_ARG;

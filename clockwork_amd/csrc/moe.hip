@@ -3,7 +3,8 @@
 //
 //   1. moe_route:  z = router x in float32, r = 1 / (1 + exp(-z)) (or softmax over the experts),
 //                  the ``top`` largest r, chosen by their z (the lower index first among equals), optionally
-//                  divided by their sum. One workgroup a token. Options: a ``correction`` per
+//                  divided by their sum. One workgroup a token. Options: a ``bias`` per expert joins
+//                  its logit; a ``correction`` per
 //                  expert joins r for the CHOICE only (the weights stay r); experts in ``groups``
 //                  equal runs of neighbours, a run scored by the sum of its ``group_top`` largest
 //                  choice scores, and only experts of the ``groups_kept`` best runs can be chosen;
@@ -50,6 +51,7 @@ typedef __attribute__((ext_vector_type(4))) unsigned int u32x4_t;
 #define MOE_MAX_EXTRA 8
 #define MOE_MAX_GROUP_TOP 64
 struct MoeRouteOptions {
+  const float* bias;        // [E] joins the logits, or null
   const float* correction;  // [E] or null
   int groups, groups_kept, group_top;   // groups <= 1: every expert can be chosen
   int extra;                // rows behind the router's E
@@ -97,7 +99,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const T* __restrict__ x
       for (int j = lane; j < H; j += 64) s += cw_to_float(xr[j]) * cw_to_float(w[j]);
     }
     s = cw_wave_sum(s);
-    if (lane == 0) r[e] = s;
+    if (lane == 0) r[e] = (opt.bias && e < E) ? s + opt.bias[e] : s;
   }
   __syncthreads();
   if (wave != 0) return;
@@ -661,14 +663,14 @@ CW_EXPORT int cw_moe_max_tiles(int n_pairs, int E, int tile_rows) {
 }
 
 CW_EXPORT int cw_moe_route(const void* x, const void* router, int dtype, int T, int H, int E, int top, int kind, int renorm,
-                           int* choice, float* score, const float* correction, int groups, int groups_kept, int group_top,
-                           int extra, float* extra_out, float renorm_eps, float scale, hipStream_t stream) {
+                           int* choice, float* score, const float* bias, const float* correction, int groups, int groups_kept,
+                           int group_top, int extra, float* extra_out, float renorm_eps, float scale, hipStream_t stream) {
   if (T < 0 || H <= 0 || E <= 0 || top <= 0 || top > E || !x || !router || !choice || !score) return CW_ERR_ARG;
   if (extra < 0 || extra > MOE_MAX_EXTRA || (extra > 0 && !extra_out)) return CW_ERR_ARG;
   if (groups > 1 && (E % groups || groups_kept < 1 || groups_kept > groups || group_top < 1 || group_top > MOE_MAX_GROUP_TOP ||
                      (E / groups) * groups_kept < top))
     return CW_ERR_ARG;
-  const MoeRouteOptions opt = {correction, groups, groups_kept, group_top, extra, extra_out, renorm, renorm_eps, scale};
+  const MoeRouteOptions opt = {bias, correction, groups, groups_kept, group_top, extra, extra_out, renorm, renorm_eps, scale};
   if (kind != MOE_ROUTER_SIGMOID && kind != MOE_ROUTER_SOFTMAX) return CW_ERR_ARG;
   if (E > MOE_MAX_EXPERTS) return CW_ERR_SIZE;
   if (T == 0) return CW_OK;

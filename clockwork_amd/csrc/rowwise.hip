@@ -7,7 +7,8 @@
 // the rotation of one part of every head, the RMS norm of a branch's output as it joins the
 // stream, the RMS norm of the stream with a weight kept as a distance from a constant, the RMS
 // norm of every query / key vector with rotation and cache write, squared ReLU, a scale, the RMS
-// norm of the scaled stream plus a branch (norms behind the residual sum), and an embedding with a
+// norm of the scaled stream plus a branch (norms behind the residual sum), Dynamic Tanh of a branch as it
+// joins and of the stream behind it, and an embedding with a
 // row for the token and the one before it.
 // Statistics, gates and the residual stream are float32; T is the activation type.
 #include "common.h"
@@ -473,31 +474,32 @@ CW_EXPORT int cw_gelu(void* x, int dtype, int64_t n, int form, hipStream_t strea
 }
 
 // ---------------------------------------------------------------- a * sigmoid(z), in place on a
-// a[t, j] <- a[t, j] / (1 + exp(-z[t, z_off + j / group])), j < n; z rows are z_stride elements
-// apart. group 1: a gate an element; group g: one gate for every run of g elements (a head).
+// a[t, j] <- a[t, j] / (1 + exp(-z[t, z_off + j / group])), j < n; a's rows are a_stride elements
+// apart, z's z_stride. group 1: a gate an element; group g: one gate for every run of g elements (a head).
 template <typename T>
-__global__ void sigmoid_mul_kernel(T* __restrict__ a, const T* __restrict__ z, int64_t z_stride, int z_off, int n,
+__global__ void sigmoid_mul_kernel(T* __restrict__ a, int64_t a_stride, const T* __restrict__ z, int64_t z_stride, int z_off, int n,
                                    int group, int64_t total) {
   for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
     const int64_t t = i / n;
     const int j = (int)(i % n) / group;
     const float g = 1.0f / (1.0f + expf(-cw_to_float(z[t * z_stride + z_off + j])));
-    a[i] = cw_from_float<T>(cw_to_float(a[i]) * g);
+    T* at = a + t * a_stride + (i - t * n);
+    *at = cw_from_float<T>(cw_to_float(*at) * g);
   }
 }
 
-CW_EXPORT int cw_sigmoid_mul(void* a, const void* z, int dtype, int64_t z_stride, int z_off, int T, int n, int group,
+CW_EXPORT int cw_sigmoid_mul(void* a, int64_t a_stride, const void* z, int dtype, int64_t z_stride, int z_off, int T, int n, int group,
                              hipStream_t stream) {
-  if (T < 0 || n <= 0 || group <= 0 || n % group || z_off < 0 || z_off + n / group > z_stride) return CW_ERR_ARG;
+  if (T < 0 || n <= 0 || a_stride < n || group <= 0 || n % group || z_off < 0 || z_off + n / group > z_stride) return CW_ERR_ARG;
   if (T == 0) return CW_OK;
   const int64_t total = (int64_t)T * n;
   int64_t blocks = (total + 255) / 256;
   if (blocks > 262144) blocks = 262144;
   dim3 grid((unsigned)blocks), block(256);
   if (dtype == CW_F32)
-    hipLaunchKernelGGL(sigmoid_mul_kernel<float>, grid, block, 0, stream, (float*)a, (const float*)z, z_stride, z_off, n, group, total);
+    hipLaunchKernelGGL(sigmoid_mul_kernel<float>, grid, block, 0, stream, (float*)a, a_stride, (const float*)z, z_stride, z_off, n, group, total);
   else if (dtype == CW_BF16)
-    hipLaunchKernelGGL(sigmoid_mul_kernel<bf16_t>, grid, block, 0, stream, (bf16_t*)a, (const bf16_t*)z, z_stride, z_off, n, group, total);
+    hipLaunchKernelGGL(sigmoid_mul_kernel<bf16_t>, grid, block, 0, stream, (bf16_t*)a, a_stride, (const bf16_t*)z, z_stride, z_off, n, group, total);
   else return CW_ERR_DTYPE;
   return cw_launch_status();
 }
@@ -1315,6 +1317,80 @@ CW_EXPORT int cw_post_norm(float* resid, const void* branch, const float* parts,
   else if (dtype == CW_BF16 && w_dtype == CW_F32) CW_BY_ROW(bf16_t, float);
   else return CW_ERR_DTYPE;
 #undef CW_BY_ROW
+#undef CW_LAUNCH
+  return cw_launch_status();
+}
+
+// ---------------------------------------------------------------- a normed branch joins, Dynamic Tanh of the stream
+//   x = resid[t, :] + (tanh(balpha * branch) * bw + bb);  resid[t, :] = x;  out = tanh(alpha * x) * w + b
+// for blocks with a Dynamic Tanh norm before and behind each sublayer: the norm behind one sublayer, the
+// residual sum and the norm ahead of the next in one kernel. branch is one of what PostBranch knows (a
+// row, float32 planes, a routed feed-forward's pairs). With ``rows`` only those rows are produced and resid
+// is left alone. out may be null (the branch only joins). float32 inside.
+template <typename T, typename WT, int N>
+__global__ __launch_bounds__(256) void join_dyt_kernel(float* __restrict__ resid, PostBranch<T> br, const WT* __restrict__ bw,
+                                                       const WT* __restrict__ bb, const float* __restrict__ balpha,
+                                                       const WT* __restrict__ w, const WT* __restrict__ b,
+                                                       const float* __restrict__ alpha, T* __restrict__ out,
+                                                       const int* __restrict__ rows, int64_t plane, int H) {
+  const int64_t i = blockIdx.x;
+  const int64_t t = rows ? (int64_t)rows[i] : i;
+  const float ba = balpha[0], a = out ? alpha[0] : 0.0f;
+  float* x = resid + t * H;
+  for (int j = (blockIdx.y * 256 + threadIdx.x) * N; j < H; j += gridDim.y * 256 * N) {
+    float v[N], r[N], y[N];
+    PostBranch<T>::load(x + j, r);
+#pragma unroll
+    for (int u = 0; u < N; ++u) v[u] = y[u] = 0.0f;
+    br.add(v, y, t, plane, j, H);
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+      float z = tanhf(ba * v[u]) * cw_to_float(bw[j + u]);
+      if (bb) z += cw_to_float(bb[j + u]);
+      v[u] = r[u] + z;
+    }
+    if (!rows) {
+      if constexpr (N == 4) store4(x + j, v); else x[j] = v[0];
+    }
+    if (!out) continue;
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+      y[u] = tanhf(a * v[u]) * cw_to_float(w[j + u]);
+      if (b) y[u] += cw_to_float(b[j + u]);
+    }
+    if constexpr (N == 4) store4(out + i * H + j, y); else out[i * H + j] = cw_from_float<T>(y[0]);
+  }
+}
+
+CW_EXPORT int cw_join_dyt(float* resid, const void* branch, const float* parts, int n_parts, const void* pairs, const int* choice,
+                          const float* score, const void* always, int top, int experts, const void* bw, const void* bb,
+                          const float* balpha, const void* w, const void* b, const float* alpha, int w_dtype, void* out, int dtype,
+                          const int* rows, int n, int T, int H, hipStream_t stream) {
+  if (T < 0 || n < 0 || H <= 0 || !resid || !bw || !balpha || (out && (!w || !alpha)) || (rows && !out)) return CW_ERR_ARG;
+  if ((branch != nullptr) + (parts != nullptr) + (pairs != nullptr) != 1) return CW_ERR_ARG;
+  if (parts && n_parts < 1) return CW_ERR_ARG;
+  if (pairs && (!choice || !score || top < 1 || experts < 0)) return CW_ERR_ARG;
+  if (n == 0) return CW_OK;
+  const int align = dtype == CW_BF16 ? 8 : 16;
+  const bool vec = H % 4 == 0 && !(((uintptr_t)resid | (uintptr_t)parts) & 15) &&
+                   !(((uintptr_t)branch | (uintptr_t)pairs | (uintptr_t)always | (uintptr_t)out) & (align - 1));
+  // few rows: a row is shared by workgroups, so that every thread has one step of its loop
+  const int per = vec ? 1024 : 256;
+  const dim3 grid(n, n <= 64 ? (H + per - 1) / per : 1), block(256);
+#define CW_LAUNCH(T_, WT_)                                                                                              \
+  do {                                                                                                                  \
+    PostBranch<T_> br{(const T_*)branch, parts, n_parts, (const T_*)pairs, choice, score, (const T_*)always, top, experts}; \
+    if (vec)                                                                                                            \
+      hipLaunchKernelGGL((join_dyt_kernel<T_, WT_, 4>), grid, block, 0, stream, resid, br, (const WT_*)bw, (const WT_*)bb, balpha, \
+                         (const WT_*)w, (const WT_*)b, alpha, (T_*)out, rows, (int64_t)T * H, H);                       \
+    else                                                                                                                \
+      hipLaunchKernelGGL((join_dyt_kernel<T_, WT_, 1>), grid, block, 0, stream, resid, br, (const WT_*)bw, (const WT_*)bb, balpha, \
+                         (const WT_*)w, (const WT_*)b, alpha, (T_*)out, rows, (int64_t)T * H, H);                       \
+  } while (0)
+  if (dtype == CW_F32 && w_dtype == CW_F32) CW_LAUNCH(float, float);
+  else if (dtype == CW_BF16 && w_dtype == CW_BF16) CW_LAUNCH(bf16_t, bf16_t);
+  else if (dtype == CW_BF16 && w_dtype == CW_F32) CW_LAUNCH(bf16_t, float);
+  else return CW_ERR_DTYPE;
 #undef CW_LAUNCH
   return cw_launch_status();
 }

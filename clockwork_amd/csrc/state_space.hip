@@ -9,7 +9,7 @@
 //
 // Single tokens (every request of the step has one): ss_step_kernel makes the convolution, the state
 // update and the output of one (request, head) in one launch. Any other step:
-//   ss_conv_kernel         the convolution of runs of a request's tokens, 16 a work item,
+//   short_conv_kernel      the convolution of runs of a request's tokens, 16 a work item,
 //   ss_chunk_state_kernel  per (chunk of tokens, head) what the chunk adds to the state,
 //                          sum over t of exp(cum_last - cum_t) d_t B_t x_t^T, and its decay exp(cum_last),
 //                          cum the running sum of the logarithms of the decays,
@@ -23,13 +23,13 @@
 // state as 16x16x4 float32 ones. Steps, decays, their logarithms, the state and the norm are float32
 // whatever the activation type T is.
 #include "common.h"
+#include "short_conv.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
 typedef __attribute__((ext_vector_type(4))) float f32x4_t;
 typedef __attribute__((ext_vector_type(4))) unsigned int u32x4_t;
 
-#define SS_CONV_TOKENS 16
-#define SS_MAX_TAPS (SS_CONV_TOKENS + 1)
+#define SS_MAX_TAPS SHORT_CONV_MAX_TAPS
 #define SS_MAX_DIM 256          // N and P
 #define SS_STEP_AHEAD 8         // rows of the state a thread of ss_step_kernel asks for at once
 
@@ -57,116 +57,6 @@ struct SsParams {
   int heads, groups, N, P, taps, channels;
 };
 
-__device__ __forceinline__ float ss_softplus(float z) { return z > 0.0f ? z + log1pf(expf(-z)) : log1pf(expf(z)); }
-__device__ __forceinline__ float ss_silu(float z) { return z / (1.0f + expf(-z)); }
-
-template <typename T, int V> struct SsVec;   // V neighbouring elements as float32
-template <typename T> struct SsVec<T, 1> {
-  static __device__ __forceinline__ void load(const T* p, float (&o)[1]) { o[0] = cw_to_float(p[0]); }
-  static __device__ __forceinline__ void store(T* p, const float (&v)[1]) { p[0] = cw_from_float<T>(v[0]); }
-};
-template <> struct SsVec<float, 4> {
-  static __device__ __forceinline__ void load(const float* p, float (&o)[4]) {
-    const float4 v = *reinterpret_cast<const float4*>(p);
-    o[0] = v.x; o[1] = v.y; o[2] = v.z; o[3] = v.w;
-  }
-  static __device__ __forceinline__ void store(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
-};
-template <> struct SsVec<bf16_t, 4> {
-  static __device__ __forceinline__ void load(const bf16_t* p, float (&o)[4]) {
-    const uint2 d = *reinterpret_cast<const uint2*>(p);
-    o[0] = __uint_as_float(d.x << 16); o[1] = __uint_as_float(d.x & 0xffff0000u);
-    o[2] = __uint_as_float(d.y << 16); o[3] = __uint_as_float(d.y & 0xffff0000u);
-  }
-  static __device__ __forceinline__ void store(bf16_t* p, const float (&v)[4]) {
-    *reinterpret_cast<uint2*>(p) = make_uint2((uint32_t)cw_float_to_bf16_bits(v[0]) | ((uint32_t)cw_float_to_bf16_bits(v[1]) << 16),
-                                              (uint32_t)cw_float_to_bf16_bits(v[2]) | ((uint32_t)cw_float_to_bf16_bits(v[3]) << 16));
-  }
-};
-
-// ---------------------------------------------------------------- the convolution of a portion
-// A thread owns V channels of an item's tokens. The workgroup of a request's first item alone reads
-// the slot's inputs, and afterwards writes the portion's last taps - 1 ones there (a thread what it has
-// read itself). TAPS 0: any number up to SS_MAX_TAPS, V = 1.
-template <typename T, int V, int TAPS>
-__global__ __launch_bounds__(256) void ss_conv_kernel(SsParams p) {
-  const int* item = p.items + 4 * (int64_t)blockIdx.x;
-  const int req = item[0], tok0 = item[1];
-  const int row0 = p.cu_q[req], q_len = p.cu_q[req + 1] - row0;
-  if (tok0 >= q_len) return;  // an item past the request's tokens (a batch of fixed shape)
-  const int ntok = min(min(item[2], SS_CONV_TOKENS), q_len - tok0);
-  const int c = (blockIdx.y * 256 + threadIdx.x) * V;
-  if (c >= p.channels) return;
-  const int slot = p.state_slots[req];
-  const bool has_slot = slot >= 0 && slot < p.n_slots;
-  float* ring = has_slot ? p.state + slot * p.state_stride + (int64_t)p.heads * p.N * p.P : nullptr;
-  const int pos0 = p.ctx_lens[req] - q_len;
-  const int taps = TAPS ? TAPS : p.taps;
-  const T* in = (const T*)p.proj + (int64_t)row0 * p.stride + p.c_off + c;
-  T* out = (T*)p.xbc + (int64_t)row0 * p.channels + c;
-  // the input of the request's token i of this portion (negative: before it, from the slot)
-  auto input = [&](int i, float (&o)[V]) __attribute__((always_inline)) {
-    if (i >= 0) {
-      SsVec<T, V>::load(in + (int64_t)i * p.stride, o);
-    } else {
-      const int pos = pos0 + i;
-#pragma unroll
-      for (int v = 0; v < V; ++v) o[v] = (pos >= 0 && ring) ? ring[(int64_t)(pos % taps) * p.channels + c + v] : 0.0f;
-    }
-  };
-  if constexpr (TAPS > 0) {
-    float w[TAPS][V], b[V], win[TAPS][V];
-#pragma unroll
-    for (int v = 0; v < V; ++v) {
-      b[v] = p.conv_b[c + v];
-#pragma unroll
-      for (int k = 0; k < TAPS; ++k) w[k][v] = p.conv_w[(int64_t)(c + v) * TAPS + k];
-    }
-#pragma unroll
-    for (int k = 0; k < TAPS - 1; ++k) input(tok0 - (TAPS - 1) + k, win[k + 1]);
-    // all of the item's rows are asked for before the first is used
-    float x[SS_CONV_TOKENS][V];
-#pragma unroll
-    for (int i = 0; i < SS_CONV_TOKENS; ++i) SsVec<T, V>::load(in + (int64_t)(tok0 + min(i, ntok - 1)) * p.stride, x[i]);
-#pragma unroll
-    for (int i = 0; i < SS_CONV_TOKENS; ++i) {
-#pragma unroll
-      for (int k = 0; k < TAPS - 1; ++k)
-#pragma unroll
-        for (int v = 0; v < V; ++v) win[k][v] = win[k + 1][v];
-      float o[V];
-#pragma unroll
-      for (int v = 0; v < V; ++v) {
-        win[TAPS - 1][v] = x[i][v];
-        float s = b[v];
-#pragma unroll
-        for (int k = 0; k < TAPS; ++k) s += w[k][v] * win[k][v];
-        o[v] = ss_silu(s);
-      }
-      if (i < ntok) SsVec<T, V>::store(out + (int64_t)(tok0 + i) * p.channels, o);
-    }
-  } else {
-    for (int i = 0; i < ntok; ++i) {
-      float o[V];
-      o[0] = p.conv_b[c];
-      for (int k = 0; k < taps; ++k) {
-        float u[V];
-        input(tok0 + i - (taps - 1) + k, u);
-        o[0] += p.conv_w[(int64_t)c * taps + k] * u[0];
-      }
-      o[0] = ss_silu(o[0]);
-      SsVec<T, V>::store(out + (int64_t)(tok0 + i) * p.channels, o);
-    }
-  }
-  if (tok0 == 0 && ring) {
-    for (int i = max(0, q_len - (taps - 1)); i < q_len; ++i) {
-      float u[V];
-      SsVec<T, V>::load(in + (int64_t)i * p.stride, u);
-#pragma unroll
-      for (int v = 0; v < V; ++v) ring[(int64_t)((pos0 + i) % taps) * p.channels + c + v] = u[v];
-    }
-  }
-}
 
 // ---------------------------------------------------------------- chunks
 // Rows of a chunk's operand in LDS: ``width`` elements of T, zeros past the operand's ``n`` and past
@@ -196,7 +86,7 @@ __device__ __forceinline__ void ss_stage(T* dst, int dst_stride, int width, cons
 // The chunk's steps and the running sum of its decays' logarithms, by the first wave (a lane a token).
 __device__ __forceinline__ void ss_steps(const SsParams& p, float raw, bool live, int h, float* dd, float* cum, int rows) {
   const int lane = threadIdx.x;
-  const float d = live ? ss_softplus(raw + p.dt_bias[h]) : 0.0f;
+  const float d = live ? cw_softplus(raw + p.dt_bias[h]) : 0.0f;
   float c = -expf(p.a_log[h]) * d;
 #pragma unroll
   for (int off = 1; off < 64; off <<= 1) {
@@ -282,7 +172,7 @@ __global__ __launch_bounds__(256) void ss_carry_kernel(SsParams p) {
   if (e >= NP || slot < 0 || slot >= p.n_slots || q_len <= 0) return;
   float* st = p.state + slot * p.state_stride + h * NP + e;
   float S[V];
-  SsVec<float, V>::load(st, S);
+  CwVec<float, V>::load(st, S);
   const int begin = p.req_first[r];
   int end = p.req_first[r + 1];
   while (end > begin && p.items[4 * (end - 1) + 1] >= q_len) --end;   // chunks past the request's tokens (a batch of fixed shape)
@@ -292,19 +182,19 @@ __global__ __launch_bounds__(256) void ss_carry_kernel(SsParams p) {
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
       const int c = min(c0 + u, end - 1);
-      SsVec<float, V>::load(p.added + ((int64_t)c * p.heads + h) * NP + e, add[u]);
+      CwVec<float, V>::load(p.added + ((int64_t)c * p.heads + h) * NP + e, add[u]);
       dec[u] = p.chunk_decay[(int64_t)c * p.heads + h];
     }
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
       if (c0 + u < end) {
-        SsVec<float, V>::store(p.added + ((int64_t)(c0 + u) * p.heads + h) * NP + e, S);
+        CwVec<float, V>::store(p.added + ((int64_t)(c0 + u) * p.heads + h) * NP + e, S);
 #pragma unroll
         for (int v = 0; v < V; ++v) S[v] = dec[u] * S[v] + add[u][v];
       }
     }
   }
-  SsVec<float, V>::store(st, S);
+  CwVec<float, V>::store(st, S);
 }
 
 // C . B of 16 tokens against 16 tokens
@@ -461,8 +351,8 @@ __global__ __launch_bounds__(256) void ss_step_kernel(SsParams p, int PW) {
   float ahead[SS_STEP_AHEAD][V];
 #pragma unroll
   for (int i = 0; i < SS_STEP_AHEAD; ++i)
-    if (active && n0 + i * rows_at_once < N) SsVec<float, V>::load(st + (int64_t)(n0 + i * rows_at_once) * P + pc, ahead[i]);
-  const float d = ss_softplus(cw_to_float(in[p.d_off + h]) + p.dt_bias[h]);
+    if (active && n0 + i * rows_at_once < N) CwVec<float, V>::load(st + (int64_t)(n0 + i * rows_at_once) * P + pc, ahead[i]);
+  const float d = cw_softplus(cw_to_float(in[p.d_off + h]) + p.dt_bias[h]);
   const float decay = expf(-expf(p.a_log[h]) * d);
   for (int e = tid; e < pw + 2 * N; e += 256) {
     // channels: this workgroup's of x, then B and C of the group
@@ -479,7 +369,7 @@ __global__ __launch_bounds__(256) void ss_step_kernel(SsParams p, int PW) {
     s += w[taps - 1] * now;
     if (mine) ring[(int64_t)(pos % taps) * p.channels + c] = now;
     // rounded as the convolution of a portion stores it
-    const float o = cw_to_float(cw_from_float<T>(ss_silu(s)));
+    const float o = cw_to_float(cw_from_float<T>(cw_silu(s)));
     if (e < pw) Xs[e] = o;
     else if (e < pw + N) Bs[e - pw] = o;
     else Cs[e - pw - N] = o;
@@ -503,21 +393,21 @@ __global__ __launch_bounds__(256) void ss_step_kernel(SsParams p, int PW) {
           S[v] = decay * ahead[i][v] + b * x[v];
           acc[v] += cc * S[v];
         }
-        SsVec<float, V>::store(st + (int64_t)n * P + pc, S);
+        CwVec<float, V>::store(st + (int64_t)n * P + pc, S);
       }
     }
 #pragma unroll 4
     for (int n = n0 + SS_STEP_AHEAD * rows_at_once; n < N; n += rows_at_once) {
       float S[V];
       float* at = st + (int64_t)n * P + pc;
-      SsVec<float, V>::load(at, S);
+      CwVec<float, V>::load(at, S);
       const float b = Bs[n], cc = Cs[n];
 #pragma unroll
       for (int v = 0; v < V; ++v) {
         S[v] = decay * S[v] + b * x[v];
         acc[v] += cc * S[v];
       }
-      SsVec<float, V>::store(at, S);
+      CwVec<float, V>::store(at, S);
     }
   }
 #pragma unroll
@@ -533,7 +423,8 @@ __global__ __launch_bounds__(256) void ss_step_kernel(SsParams p, int PW) {
 // ---------------------------------------------------------------- gate and norm
 // out[t, j] = v_j / sqrt(mean over j's part of v^2 + eps) * w[j] with v = y silu(z); the row's ``n``
 // elements lie in ``parts`` equal parts. Parts of up to 512 elements are a wave's, larger ones the workgroup's.
-template <typename T, int V>
+// GATE_LAST: v = y, and what is normed and weighted is multiplied by the logistic function of z.
+template <typename T, int V, bool GATE_LAST>
 __global__ __launch_bounds__(256) void gated_parts_norm_kernel(const float* __restrict__ y, const T* __restrict__ z,
                                                                int64_t z_stride, const float* __restrict__ w, float eps,
                                                                T* __restrict__ out, int n, int parts) {
@@ -546,11 +437,12 @@ __global__ __launch_bounds__(256) void gated_parts_norm_kernel(const float* __re
   const float* yr = y + t * n;
   const T* zr = z + t * z_stride;
   auto value = [&](int j, float (&v)[V]) __attribute__((always_inline)) {
+    CwVec<float, V>::load(yr + j, v);
+    if (GATE_LAST) return;
     float g[V];
-    SsVec<float, V>::load(yr + j, v);
-    SsVec<T, V>::load(zr + j, g);
+    CwVec<T, V>::load(zr + j, g);
 #pragma unroll
-    for (int i = 0; i < V; ++i) v[i] *= ss_silu(g[i]);
+    for (int i = 0; i < V; ++i) v[i] *= cw_silu(g[i]);
   };
   for (int q = first; q < parts; q += step) {
     float ss = 0.0f;
@@ -573,7 +465,13 @@ __global__ __launch_bounds__(256) void gated_parts_norm_kernel(const float* __re
       value(j, v);
 #pragma unroll
       for (int i = 0; i < V; ++i) v[i] *= inv * w[j + i];
-      SsVec<T, V>::store(out + t * n + j, v);
+      if (GATE_LAST) {
+        float g[V];
+        CwVec<T, V>::load(zr + j, g);
+#pragma unroll
+        for (int i = 0; i < V; ++i) v[i] *= cw_logistic(g[i]);
+      }
+      CwVec<T, V>::store(out + t * n + j, v);
     }
   }
 }
@@ -667,25 +565,11 @@ CW_EXPORT int cw_state_space_chunks(int dtype, const void* proj, int64_t stride,
   if (n_requests == 0 || n_chunks == 0) return CW_OK;
   const int elem = dtype == CW_BF16 ? 2 : 4, Q = cw_state_space_chunk(dtype, N, P);
   p.xbc = xbc;
-  p.items = conv_items;
   {
-    const bool v4 = p.channels % 4 == 0 && stride % 4 == 0 && c_off % 4 == 0 && !(((uintptr_t)proj | (uintptr_t)xbc) & (elem * 4 - 1)) &&
-                    taps >= 2 && taps <= 4;
-    const int per = v4 ? 4 : 1;
-    dim3 grid(n_conv_items, (p.channels + 256 * per - 1) / (256 * per)), block(256);
-#define CW_CONV(T_, V_, K_) hipLaunchKernelGGL((ss_conv_kernel<T_, V_, K_>), grid, block, 0, stream, p)
-#define CW_BY_TAPS(T_)                    \
-  do {                                    \
-    if (!v4) CW_CONV(T_, 1, 0);           \
-    else if (taps == 2) CW_CONV(T_, 4, 2); \
-    else if (taps == 3) CW_CONV(T_, 4, 3); \
-    else CW_CONV(T_, 4, 4);               \
-  } while (0)
-    if (dtype == CW_F32) CW_BY_TAPS(float);
-    else CW_BY_TAPS(bf16_t);
-#undef CW_BY_TAPS
-#undef CW_CONV
-    if (hipGetLastError() != hipSuccess) return CW_ERR_LAUNCH;
+    const ShortConv c = {proj, stride, c_off, xbc, p.channels, 0, conv_w, conv_b, 1, state, state_stride, (int64_t)heads * N * P,
+                         n_slots, state_slots, cu_q, ctx_lens, conv_items, p.channels, taps};
+    const int rc2 = short_conv_launch(c, dtype, n_conv_items, stream);
+    if (rc2 != CW_OK) return rc2;
   }
   p.items = chunk_items;
   p.req_first = req_first;
@@ -725,15 +609,20 @@ CW_EXPORT int cw_state_space_chunks(int dtype, const void* proj, int64_t stride,
 }
 
 CW_EXPORT int cw_gated_parts_norm(const float* y, const void* z, int dtype, int64_t z_stride, int z_off, const float* w, float eps,
-                                  void* out, int T, int n, int parts, hipStream_t stream) {
+                                  void* out, int T, int n, int parts, int gate_last, hipStream_t stream) {
   if (T < 0 || n < 1 || parts < 1 || n % parts || !y || !z || !w || !out || z_off < 0 || z_off + n > z_stride) return CW_ERR_ARG;
   if (T == 0) return CW_OK;
   const int elem = dtype == CW_BF16 ? 2 : 4;
   const bool v4 = (n / parts) % 4 == 0 && z_stride % 4 == 0 && z_off % 4 == 0 && !(((uintptr_t)z | (uintptr_t)out) & (elem * 4 - 1)) &&
                   !((uintptr_t)y & 15);
   dim3 grid(T), block(256);
-#define CW_LAUNCH(T_, V_) \
-  hipLaunchKernelGGL((gated_parts_norm_kernel<T_, V_>), grid, block, 0, stream, y, (const T_*)z + z_off, z_stride, w, eps, (T_*)out, n, parts)
+#define CW_LAUNCH(T_, V_)                                                                                                        \
+  do {                                                                                                                           \
+    if (gate_last)                                                                                                               \
+      hipLaunchKernelGGL((gated_parts_norm_kernel<T_, V_, true>), grid, block, 0, stream, y, (const T_*)z + z_off, z_stride, w, eps, (T_*)out, n, parts); \
+    else                                                                                                                         \
+      hipLaunchKernelGGL((gated_parts_norm_kernel<T_, V_, false>), grid, block, 0, stream, y, (const T_*)z + z_off, z_stride, w, eps, (T_*)out, n, parts); \
+  } while (0)
   if (dtype == CW_F32) { if (v4) CW_LAUNCH(float, 4); else CW_LAUNCH(float, 1); }
   else if (dtype == CW_BF16) { if (v4) CW_LAUNCH(bf16_t, 4); else CW_LAUNCH(bf16_t, 1); }
   else return CW_ERR_DTYPE;

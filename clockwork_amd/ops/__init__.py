@@ -129,7 +129,7 @@ def _declare(name: str, lib: ctypes.CDLL) -> None:
             "cw_qk_rownorm_store": [P, I, L, I, I, I, I, I, I, P, P, I, F, P, P, P, L, I, P],
             "cw_add_dyt": [P, P, I, F, P, P, P, I, P, P, I, P, I, I, P],
             "cw_gelu": [P, I, L, I, P],
-            "cw_sigmoid_mul": [P, P, I, L, I, I, I, I, P],
+            "cw_sigmoid_mul": [P, L, P, I, L, I, I, I, I, P],
             "cw_bias_store": [P, I, L, I, I, I, I, I, I, P, I, P, P, P, L, I, P],
             "cw_latent_store": [P, I, L, I, I, I, I, I, I, I, P, P, I, F, P, P, P, P, P, I, I, L, I, P],
             "cw_rotate_part": [P, I, L, L, I, P, L, L, I, I, I, I, I, I, P, P, I, P],
@@ -141,6 +141,7 @@ def _declare(name: str, lib: ctypes.CDLL) -> None:
             "cw_stream_beside_input": [P, P, P, P, P, I, I, I, I, I, P],
             "cw_relu_squared": [P, I, L, P],
             "cw_scale": [P, L, F, P],
+            "cw_join_dyt": [P, P, P, I, P, P, P, P, I, I, P, P, P, P, P, P, I, P, I, P, I, I, I, P],
             "cw_post_norm": [P, P, P, I, P, P, P, P, I, I, F, P, I, F, F, P, I, I, I, P],
             "cw_embedding_pair": [P, I, P, F, P, I, L, L, P, I, P, P, I, P, I, I, I, P],
         },
@@ -151,12 +152,32 @@ def _declare(name: str, lib: ctypes.CDLL) -> None:
             "cw_state_space_workspace_floats": [I, I, I, I],
             "cw_state_space_step": [I, P, L, I, I, I, P, P, P, P, P, P, L, I, P, P, P, P, I, I, I, I, I, I, I, P],
             "cw_state_space_chunks": [I, P, L, I, I, I, P, P, P, P, P, P, L, I, P, P, P, P, P, P, I, P, I, P, P, I, I, I, I, I, I, P],
-            "cw_gated_parts_norm": [P, P, I, L, I, P, F, P, I, I, I, P],
+            "cw_gated_parts_norm": [P, P, I, L, I, P, F, P, I, I, I, I, P],
+        },
+        "short_conv": {
+            "cw_short_conv_tokens": [],
+            "cw_short_conv_max_taps": [],
+            "cw_short_conv": [I, P, L, I, P, L, P, P, I, P, L, L, I, P, P, P, P, I, I, I, P],
+            "cw_qkv_conv_run": [I, I, I, I],
+            "cw_qkv_conv_store": [I, P, L, I, I, I, I, I, P, I, P, L, L, I, P, P, P, P, I, P, P, F, P, P, I, F, F, P, P, P, P, L, P],
+        },
+        "selective_scan": {
+            "cw_selective_scan_max_segment": [I],
+            "cw_selective_scan_workspace_floats": [I, I, I, I],
+            "cw_selective_scan_step": [I, P, P, L, I, P, L, P, P, P, P, P, L, I, P, P, P, L, F, I, I, I, I, P],
+            "cw_selective_scan_segments": [I, P, P, L, I, P, L, P, P, P, P, P, L, I, P, P, P, L, F, P, I, I, P, P, I, I, I, I, I, P],
+        },
+        "matrix_memory": {
+            "cw_matrix_memory_chunk": [I, I],
+            "cw_matrix_memory_slot_floats": [I, I, I],
+            "cw_matrix_memory_workspace_floats": [I, I, I, I, I, I],
+            "cw_matrix_memory_step": [I, P, L, I, I, I, P, P, P, I, F, F, P, L, I, P, P, P, P, I, I, I, I, I, P],
+            "cw_matrix_memory_chunks": [I, P, L, I, I, I, P, P, P, I, F, F, P, L, I, P, P, P, P, P, I, P, P, I, I, I, I, I, P],
         },
         "moe": {
             "cw_moe_tile_rows": [I],
             "cw_moe_max_tiles": [I, I, I],
-            "cw_moe_route": [P, P, I, I, I, I, I, I, I, P, P, P, I, I, I, I, P, F, F, P],
+            "cw_moe_route": [P, P, I, I, I, I, I, I, I, P, P, P, P, I, I, I, I, P, F, F, P],
             "cw_moe_plan": [P, I, I, I, P, I, P, I, P, P],
             "cw_moe_expert_product": [I, I, P, P, P, I, P, P, P, I, P, I, I, I, I, F, P],
             "cw_moe_gather": [P, P, I, P, P, I, I, P, I, I, I, P],
@@ -253,6 +274,18 @@ def _gpu(*tensors) -> None:
     for t in tensors:
         if t is not None and not (t.is_cuda and t.is_contiguous()):
             raise KernelError("kernel arguments must live on the GPU and be contiguous")
+
+
+def _gpu_rows(t: torch.Tensor) -> int:
+    """A matrix on the GPU whose rows may lie apart (columns of a wider one): the elements between rows."""
+    if not (t.is_cuda and t.dim() == 2 and (t.stride(1) == 1 or t.shape[1] == 1) and (t.shape[0] <= 1 or t.stride(0) >= t.shape[1])):
+        raise KernelError("rows of a kernel's matrix must live on the GPU, each contiguous, none over another")
+    return t.stride(0) if t.shape[0] > 1 else max(t.stride(0), t.shape[1])
+
+
+def _room(t: torch.Tensor) -> int:
+    """Elements from the tensor's first one to the end of its memory."""
+    return t.untyped_storage().nbytes() // t.element_size() - t.storage_offset()
 
 
 def _i32(t, n: int | None, what: str) -> None:
@@ -435,9 +468,14 @@ def rope_kv_write(qkv, bias, positions, slots, inv_freq, rotary_dim: int, nh: in
     )
 
 
+# in the place of a clipped gated activation's limit: max(gate, 0) * up
+RELU_GATE = -1.0
+
+
 def silu_mul(gate_up: torch.Tensor, out: torch.Tensor, limit: float = 0.0) -> torch.Tensor:
     """out[t, i] = silu(gate_up[t, i]) * gate_up[t, I + i]; ``limit`` > 0: the clipped gated activation
-    g * logistic(1.702 g) * (u + 1) with g = min(gate, limit), u = up cut to [-limit, limit]."""
+    g * logistic(1.702 g) * (u + 1) with g = min(gate, limit), u = up cut to [-limit, limit];
+    ``RELU_GATE``: max(gate, 0) * up."""
     _gpu(gate_up, out)
     T, two_i = gate_up.shape
     if not (two_i % 2 == 0 and tuple(out.shape) == (T, two_i // 2) and out.dtype == gate_up.dtype):
@@ -1005,8 +1043,8 @@ def swiglu_norm_fusable(M: int, two_i: int, K: int, dtype, gate_up_weight, delta
 
 
 def linear_swiglu(x, gate_up_weight: torch.Tensor, policy: "ProductPolicy | None" = None, limit: float = 0.0) -> torch.Tensor:
-    """silu(x @ gate.T) * (x @ up.T) for gate_up_weight = [gate; up] stacked along dim 0; ``limit`` > 0:
-    the clipped gated activation (see ``silu_mul``) of the two products instead.
+    """silu(x @ gate.T) * (x @ up.T) for gate_up_weight = [gate; up] stacked along dim 0; ``limit`` > 0 or
+    ``RELU_GATE``: the other activations of the two products that ``silu_mul`` knows.
 
     Few bfloat16 rows: one kernel that streams the weights once and applies the gate in its
     epilogue. Otherwise the product followed by the gate kernel, or (``policy``, see ``linear``)
@@ -1082,7 +1120,8 @@ def attention_prefill(q, q_stride: int, out, k_cache, v_cache, block_tables, ctx
     computes all of its keys)."""
     if not (prefill_row_blocks_ok(hd, row_blocks)):
         raise KernelError(f"the kernel for head size {hd} does not take {row_blocks} row blocks")
-    _gpu(out, k_cache, v_cache, block_tables, ctx_lens, cu_q, items, workspace)
+    _gpu(k_cache, v_cache, block_tables, ctx_lens, cu_q, items, workspace)
+    out_stride = _gpu_rows(out)
     ws_floats = 0
     if workspace is not None:
         need = prefill_attention_workspace_floats(hd, n_items, nh, nkv, row_blocks)
@@ -1105,7 +1144,7 @@ def attention_prefill(q, q_stride: int, out, k_cache, v_cache, block_tables, ctx
         raise KernelError("cache must be [..., nkv, hd]")
     _check(
         _load("attention", hd).cw_attention_prefill_bf16(
-            q.data_ptr(), int(q_stride), _ptr(out), out.shape[1], _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
+            q.data_ptr(), int(q_stride), _ptr(out), out_stride, _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
             block_tables.shape[1], _ptr(ctx_lens), _ptr(cu_q), _ptr(items), n_items, nh, nkv, block_size,
             window, float(scale), _zero_row(out.device), int(row_blocks), int(workspace is not None), _ptr(workspace),
             ws_floats, float(softcap), _stream()),
@@ -1148,7 +1187,8 @@ def attention_decode(q, q_stride: int, out, k_cache, v_cache, block_tables, ctx_
     With more than one split it needs a float32 ``workspace``. ``identity``: item i is request i
     with its token in row i (no other items). ``split_keys`` > 0: every split takes that many
     keys at a fixed place; no context may then be longer than ``max_ctx`` <= n_splits * split_keys."""
-    _gpu(out, k_cache, v_cache, block_tables, ctx_lens, cu_q, items, workspace)
+    _gpu(k_cache, v_cache, block_tables, ctx_lens, cu_q, items, workspace)
+    out_stride = _gpu_rows(out)
     if not (q.is_cuda and q.dtype == out.dtype == k_cache.dtype == v_cache.dtype == torch.bfloat16):
         raise KernelError("the decode kernel is bfloat16")
     if not (out.dim() == 2 and out.shape[0] >= n_tokens and out.shape[1] == nh * hd):
@@ -1178,7 +1218,7 @@ def attention_decode(q, q_stride: int, out, k_cache, v_cache, block_tables, ctx_
         ws_floats = workspace.numel()
     _check(
         lib.cw_attention_decode_bf16(
-            q.data_ptr(), int(q_stride), _ptr(out), out.shape[1], _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
+            q.data_ptr(), int(q_stride), _ptr(out), out_stride, _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
             block_tables.shape[1], _ptr(ctx_lens), _ptr(cu_q), _ptr(items), n_items, nh, nkv, block_size, n_splits,
             window, float(scale), _ptr(workspace), ws_floats, _zero_row(out.device), int(bool(identity)),
             int(split_keys), int(max_ctx), float(softcap), _stream()),
@@ -1798,14 +1838,15 @@ def gelu_(x: torch.Tensor, form: str = "erf") -> torch.Tensor:
 
 
 def sigmoid_mul_(a: torch.Tensor, z: torch.Tensor, z_off: int, group: int = 1) -> torch.Tensor:
-    """a[t, j] <- a[t, j] * sigmoid(z[t, z_off + j // group]), in place on ``a`` [T, n]; ``z``
-    [T, width]. ``group`` 1: a gate an element; g: one gate for every run of g elements (a head)."""
-    _gpu(a, z)
+    """a[t, j] <- a[t, j] * sigmoid(z[t, z_off + j // group]), in place on ``a`` [T, n] (its rows may lie
+    apart); ``z`` [T, width]. ``group`` 1: a gate an element; g: one gate for every run of g elements (a head)."""
+    _gpu(z)
+    a_stride = _gpu_rows(a)
     T, n = a.shape
     _need(group >= 1 and n % group == 0, "the gated runs must tile the row")
     _need(z.dim() == 2 and z.shape[0] == T and z.dtype == a.dtype and 0 <= z_off and z_off + n // group <= z.shape[1],
           "the gates must be [T, width] columns of the activations' type")
-    _check(_load("rowwise").cw_sigmoid_mul(_ptr(a), _ptr(z), dtype_code(a.dtype), z.shape[1], int(z_off), T, n, int(group),
+    _check(_load("rowwise").cw_sigmoid_mul(_ptr(a), a_stride, _ptr(z), dtype_code(a.dtype), z.shape[1], int(z_off), T, n, int(group),
                                            _stream()), "sigmoid_mul")
     return a
 
@@ -1968,13 +2009,14 @@ def rows_attention(q, q_strides, out, out_strides, k_plane, v_plane, block_table
     (``rows_mfma_supported``; items of up to ``ROWS_MFMA_TOKENS`` tokens), every item's keys cut
     into ``key_runs`` runs that a second kernel puts together."""
     alias = v_plane is None
-    _gpu(q, out, k_plane, v_plane, block_tables, ctx_lens, cu_q, items, sink, lam)
+    _gpu(q, k_plane, v_plane, block_tables, ctx_lens, cu_q, items, sink, lam)
+    _need(out.is_cuda and (out.is_contiguous() or (out.dim() == 2 and out.stride(1) == 1)), "the output must live on the GPU, its rows contiguous")
     qs, qh = int(q_strides[0]), int(q_strides[1])
     os_, oh = int(out_strides[0]), int(out_strides[1])
     _need(out.dtype == q.dtype, "queries and output differ in type")
     # the furthest element a token row of the step can touch must lie inside the tensors
     def _fits(t, tok_stride, head_stride, width, tokens):
-        return tokens == 0 or (tokens - 1) * tok_stride + (heads - 1) * head_stride + width <= t.numel()
+        return tokens == 0 or (tokens - 1) * tok_stride + (heads - 1) * head_stride + width <= _room(t)
     tokens = out.numel() // (heads * vdim)
     _need(_fits(q, qs, qh, maps * dim, tokens) and _fits(out, os_, oh, vdim, tokens), "q / out strides reach outside the tensors")
     k2 = k_plane.reshape(k_plane.shape[0], -1)
@@ -2296,23 +2338,24 @@ ROUTER_KINDS = {"sigmoid": 0, "softmax": 1}
 
 
 def moe_route(x: torch.Tensor, router: torch.Tensor, top: int, kind: str = "sigmoid", renormalize: bool = False,
-              correction=None, groups=None, extra: int = 0, renorm_eps: float = 0.0, scale: float = 1.0):
+              bias=None, correction=None, groups=None, extra: int = 0, renorm_eps: float = 0.0, scale: float = 1.0):
     """(choice int32 [T, top], score float32 [T, top]): the ``top`` experts with the largest
     logistic (or softmax) of router x, the lower index first among equals, in falling order;
     ``renormalize``: the chosen scores are divided by their sum (plus ``renorm_eps``); ``scale``
     multiplies them last. float32 sums.
 
-    ``correction`` float32 [experts]: added to the scores for the choice only. ``groups``
+    ``bias`` float32 [experts]: joins the logits. ``correction`` float32 [experts]: added to the scores for the choice only. ``groups``
     (count, kept, top): the experts lie in ``count`` equal runs of neighbours, a run's score is the
     sum of its ``top`` largest choice scores, and only experts of the ``kept`` best runs can be
     chosen. ``extra`` n: the router's matrix has n more rows behind the experts' (gates that
     read the same input); their logistic values come back as a third result, float32 [T, n]."""
-    _gpu(x, router, correction)
+    _gpu(x, router, bias, correction)
     T, H = x.shape
     E = router.shape[0] - int(extra)
     _need(router.dim() == 2 and router.shape[1] == H and router.dtype == x.dtype and extra >= 0 and E >= 1,
           "the router must be [experts (+ extra), H] in x's type")
     _need(1 <= top <= E and kind in ROUTER_KINDS, f"top {top} of {E} experts, router kind {kind!r}")
+    _need(bias is None or (bias.dtype == torch.float32 and bias.numel() == E), "the router's bias must be float32 [experts]")
     _need(correction is None or (correction.dtype == torch.float32 and correction.numel() == E), "the correction must be float32 [experts]")
     count, kept, run_top = groups if groups is not None else (1, 1, 1)
     _need(count >= 1 and E % count == 0 and 1 <= kept <= count and run_top >= 1 and (E // count) * kept >= top,
@@ -2321,7 +2364,7 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, top: int, kind: str = "sigm
     score = torch.empty((T, top), dtype=torch.float32, device=x.device)
     gates = torch.empty((T, extra), dtype=torch.float32, device=x.device) if extra else None
     _check(_load("moe").cw_moe_route(_ptr(x), _ptr(router), dtype_code(x.dtype), T, H, E, top, ROUTER_KINDS[kind],
-                                     int(bool(renormalize)), _ptr(choice), _ptr(score), _ptr(correction), int(count), int(kept),
+                                     int(bool(renormalize)), _ptr(choice), _ptr(score), _ptr(bias), _ptr(correction), int(count), int(kept),
                                      int(run_top), int(extra), _ptr(gates), float(renorm_eps), float(scale), _stream()), "moe_route")
     return (choice, score, gates) if extra else (choice, score)
 
@@ -2595,14 +2638,246 @@ def state_space(proj: torch.Tensor, z_off: int, c_off: int, d_off: int, conv_w, 
     return y
 
 
-def gated_parts_norm(y: torch.Tensor, z: torch.Tensor, z_off: int, weight, eps: float, parts: int) -> torch.Tensor:
+def gated_parts_norm(y: torch.Tensor, z: torch.Tensor, z_off: int, weight, eps: float, parts: int, gate_last: bool = False) -> torch.Tensor:
     """v = y * silu(z[:, z_off:]), every one of ``parts`` equal parts of a row divided by its own root mean
-    square, times ``weight``; y and weight float32, the result in z's type."""
+    square, times ``weight``; ``gate_last``: v = y, and the logistic function of z multiplies last. y and
+    weight float32, the result in z's type."""
     _gpu(y, z, weight)
     T, n = y.shape
     _need(y.dtype == torch.float32 and weight.dtype == torch.float32 and weight.numel() == n and parts >= 1 and n % parts == 0
           and z.dim() == 2 and z.shape[0] == T and 0 <= z_off and z_off + n <= z.shape[1], "gated_parts_norm shapes")
     out = torch.empty((T, n), dtype=z.dtype, device=z.device)
     _check(_load("state_space").cw_gated_parts_norm(_ptr(y), _ptr(z), dtype_code(z.dtype), z.shape[1], int(z_off), _ptr(weight),
-                                                    float(eps), _ptr(out), T, n, int(parts), _stream()), "gated_parts_norm")
+                                                    float(eps), _ptr(out), T, n, int(parts), int(bool(gate_last)), _stream()),
+           "gated_parts_norm")
     return out
+
+
+# ---------------------------------------------------------------------------------------------
+class NormedBranch:
+    """A pending branch that passes a norm of its own as it joins the stream (``norm``: a Dynamic Tanh
+    part): what a block with a norm behind each sublayer hands to the norm that comes next."""
+
+    __slots__ = ("branch", "norm")
+
+    def __init__(self, branch, norm) -> None:
+        self.branch, self.norm = branch, norm
+
+
+def join_dynamic_tanh(resid, branch, b_weight, b_bias, b_alpha, weight=None, bias=None, alpha=None, out=None, rows=None):
+    """resid += tanh(b_alpha * branch) * b_weight + b_bias, then (``out`` not None) out = tanh(alpha * resid) *
+    weight + bias, float32 inside. ``branch``: [T, H] in the activation type, :class:`PartialSums` or
+    :class:`RoutedSum` without identity experts (both added up inside). With ``rows`` only those rows are
+    made, into out[i], and resid is left alone."""
+    parts = pairs = choice = score = always = plain = None
+    n_parts = top = experts = 0
+    T, H = resid.shape
+    _need(resid.dtype == torch.float32, "the residual stream is float32")
+    dtype = out.dtype if out is not None else None
+    if isinstance(branch, PartialSums):
+        parts = branch.parts
+        n_parts = parts.shape[0]
+        dtype = dtype or (torch.bfloat16 if b_weight.dtype == torch.bfloat16 else torch.float32)
+        _need(tuple(parts.shape) == (n_parts, T, H) and parts.dtype == torch.float32, "partial sums must be float32 [parts, T, H]")
+    elif isinstance(branch, RoutedSum):
+        pairs, choice, score, always, top, experts = branch.y, branch.choice, branch.score, branch.always, branch.top, branch.experts
+        dtype = dtype or pairs.dtype
+        _need(pairs.dtype == dtype and tuple(pairs.shape) == (T * top, H) and choice.dtype == torch.int32 and choice.numel() == T * top
+              and score.dtype == torch.float32 and score.numel() == T * top, "a routed sum has a row, a choice and a score a pair")
+        _need(always is None or (tuple(always.shape) == (T, H) and always.dtype == dtype), "the expert of every token must be [T, H]")
+    else:
+        plain = branch
+        dtype = dtype or plain.dtype
+        _need(tuple(plain.shape) == (T, H) and plain.dtype == dtype, "the branch must be [T, H] in the activation type")
+    _gpu(resid, plain, parts, pairs, choice, score, always, b_weight, b_bias, b_alpha, weight, bias, alpha, out, rows)
+    n = T if rows is None else rows.numel()
+    if rows is not None:
+        _i32(rows, n, "rows")
+        _need(out is not None, "chosen rows need an output")
+    _need(out is None or (tuple(out.shape) == (n, H) and weight is not None and alpha is not None), f"out must be [{n}, {H}]")
+    for wt in (b_weight, b_bias, weight, bias):
+        _need(wt is None or (wt.numel() == H and wt.dtype == b_weight.dtype), "norm weights and biases must have the row's size and one type")
+    for a in (b_alpha, alpha):
+        _need(a is None or (a.dtype == torch.float32 and a.numel() == 1), "alpha must be one float32 element")
+    _check(_load("rowwise").cw_join_dyt(_ptr(resid), _ptr(plain), _ptr(parts), n_parts, _ptr(pairs), _ptr(choice), _ptr(score), _ptr(always),
+                                        int(top), int(experts), _ptr(b_weight), _ptr(b_bias), _ptr(b_alpha), _ptr(weight), _ptr(bias),
+                                        _ptr(alpha), dtype_code(b_weight.dtype), _ptr(out), dtype_code(dtype), _ptr(rows), n, T, H,
+                                        _stream()), "join_dynamic_tanh")
+    return out
+
+
+# ---------------------------------------------------------------------------------------------
+def short_conv_tokens() -> int:
+    """Tokens of one request that a work item of ``short_conv`` holds."""
+    return int(_load("short_conv").cw_short_conv_tokens())
+
+
+def short_conv_max_taps() -> int:
+    return int(_load("short_conv").cw_short_conv_max_taps())
+
+
+def _step_indices(ctx_like, n_requests: int) -> None:
+    for t, n, what in ((ctx_like[0], n_requests, "state_slots"), (ctx_like[1], n_requests + 1, "cu_q"), (ctx_like[2], n_requests, "ctx_lens")):
+        if t is not None:
+            _i32(t, n, what)
+
+
+def short_conv(x: torch.Tensor, off: int, channels: int, weight, bias, state, ring_off: int, state_slots, cu_q, ctx_lens, items,
+               n_items: int, n_requests: int, silu: bool = True) -> torch.Tensor:
+    """A causal convolution of every one of ``channels`` columns of ``x`` [T, width] from ``off`` on, over each
+    request's tokens: ``weight`` float32 [channels, taps] (its last column meets the token itself), ``bias``
+    float32 [channels] or None, then silu if asked. A request's latest inputs wait in its slot of ``state``
+    (float32), from element ``ring_off`` on, [taps][channels] by position. ``items``: runs of up to
+    ``short_conv_tokens()`` tokens. Returns [T, channels]."""
+    _gpu(x, weight, bias, state, state_slots, cu_q, ctx_lens, items)
+    T, width = x.shape
+    taps = weight.shape[1]
+    _need(weight.dtype == torch.float32 and tuple(weight.shape) == (channels, taps), "the filters must be float32 [channels, taps]")
+    _need(bias is None or (bias.dtype == torch.float32 and bias.numel() == channels), "the bias must be float32 [channels]")
+    _need(0 <= off and off + channels <= width, "the convolution's columns lie outside the rows")
+    _need(state.dtype == torch.float32 and state[0].numel() >= ring_off + taps * channels, "the slot has no room for the inputs")
+    _step_indices((state_slots, cu_q, ctx_lens), n_requests)
+    _i32(items, 4 * n_items, "items")
+    out = torch.empty((T, channels), dtype=x.dtype, device=x.device)
+    _check(_load("short_conv").cw_short_conv(dtype_code(x.dtype), _ptr(x), width, int(off), _ptr(out), channels, _ptr(weight), _ptr(bias),
+                                             int(bool(silu)), _ptr(state), state[0].numel(), int(ring_off), state.shape[0],
+                                             _ptr(state_slots), _ptr(cu_q), _ptr(ctx_lens), _ptr(items), n_items, channels, taps,
+                                             _stream()), "short_conv")
+    return out
+
+
+def qkv_conv_run(nq: int, nk: int, rot_dims: int, taps: int) -> int:
+    """Tokens of one request that a work item of ``qkv_conv_store`` holds (0: beyond the kernel)."""
+    return int(_load("short_conv").cw_qkv_conv_run(nq, nk, rot_dims, taps))
+
+
+def qkv_conv_store(proj: torch.Tensor, off: int, nq: int, nk: int, nv: int, dim: int, conv, state, state_slots, cu_q, ctx_lens, items,
+                   n_items: int, n_requests: int, q_weight, k_weight, eps: float, positions, freq, rot_dims: int, rot_mult: float,
+                   v_scale: float, slots, k_plane, v_plane) -> torch.Tensor:
+    """Rows of ``proj`` [T, width] hold a token's queries (``nq`` elements), keys (``nk``) and values (``nv``) one
+    behind the other from column ``off``. A causal convolution of every channel (``conv`` float32 [nq + nk +
+    nv, taps] or None; the latest inputs in the request's slot of ``state``), an RMS norm of the whole query
+    and of the whole key projection (``q_weight``, ``k_weight`` float32, both or neither), the rotation of the
+    first ``rot_dims`` elements of every head of ``dim`` (half-split pairs, angle position * freq[i], cosine and
+    sine times ``rot_mult``); keys and ``v_scale`` times the values to the cache rows. Returns the queries
+    [T, nq]. ``items``: runs of up to ``qkv_conv_run`` tokens."""
+    _gpu(proj, conv, state, state_slots, cu_q, ctx_lens, items, q_weight, k_weight, positions, freq, slots, k_plane, v_plane)
+    T, width = proj.shape
+    C = nq + nk + nv
+    taps = 0 if conv is None else conv.shape[1]
+    _need(0 <= off and off + C <= width, "the projection's columns lie outside the rows")
+    if conv is not None:
+        _need(conv.dtype == torch.float32 and tuple(conv.shape) == (C, taps), "the filters must be float32 [channels, taps]")
+        _need(state.dtype == torch.float32 and state[0].numel() >= taps * C, "the slot has no room for the inputs")
+    _step_indices((state_slots if conv is not None else None, cu_q, ctx_lens), n_requests)
+    _i32(items, 4 * n_items, "items")
+    _i32(slots, T, "slots")
+    _need((q_weight is None) == (k_weight is None), "norm weights for queries and keys, or for neither")
+    if q_weight is not None:
+        _need(q_weight.dtype == k_weight.dtype == torch.float32 and q_weight.numel() == nq and k_weight.numel() == nk,
+              "the norms' weights must be float32 of the projections' sizes")
+    if rot_dims:
+        _i32(positions, T, "positions")
+        _need(freq is not None and freq.dtype == torch.float32 and freq.numel() >= rot_dims // 2, "freq must be float32 with rot_dims / 2 elements")
+    _need(k_plane.dtype == v_plane.dtype == proj.dtype and k_plane.numel() % nk == 0 and v_plane.numel() % nv == 0
+          and k_plane.numel() // nk == v_plane.numel() // nv, "key and value planes must hold the same number of rows")
+    q = torch.empty((T, nq), dtype=proj.dtype, device=proj.device)
+    _check(_load("short_conv").cw_qkv_conv_store(
+        dtype_code(proj.dtype), _ptr(proj), width, int(off), nq, nk, nv, int(dim), _ptr(conv), taps, _ptr(state) if conv is not None else None,
+        state[0].numel() if conv is not None else 0, 0, state.shape[0] if conv is not None else 0, _ptr(state_slots), _ptr(cu_q),
+        _ptr(ctx_lens), _ptr(items), n_items, _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(positions), _ptr(freq), int(rot_dims),
+        float(rot_mult), float(v_scale), _ptr(slots), _ptr(q), _ptr(k_plane), _ptr(v_plane), k_plane.numel() // nk, _stream()),
+        "qkv_conv_store")
+    return q
+
+
+# ---------------------------------------------------------------------------------------------
+def selective_scan_max_segment(n_state: int) -> int:
+    """The most tokens a segment of ``selective_scan`` may have with that many states a channel (0: beyond the kernels)."""
+    return int(_load("selective_scan").cw_selective_scan_max_segment(n_state))
+
+
+def selective_scan(x: torch.Tensor, z: torch.Tensor, z_off: int, low: torch.Tensor, w_dt, dt_bias, a2, skip, state, state_slots, cu_q,
+                   n_requests: int, out: torch.Tensor, out_scale: float, rank: int, segments=None) -> torch.Tensor:
+    """S <- exp(d A) S + d x B (a channel and state each), y = S . C + D x, out = y * silu(z) * out_scale for the
+    step's tokens, from and to each request's slot of ``state`` (float32, its first n_state * inner elements
+    [n_state, inner]). ``x`` [T, inner]; gates in the columns of ``z`` [T, width] from ``z_off``; rows of ``low``
+    [T, >= rank + 2 n_state] hold the step's input (``rank``), B and C; d = softplus(w_dt low + dt_bias) with
+    ``w_dt`` [inner, rank]. ``a2`` float32 [n_state, inner] is A log2(e). ``out`` [T, inner], its rows may lie apart.
+
+    ``segments`` None: every request has one token. Else (items, their number, tokens of a segment, first
+    segment of each request)."""
+    _gpu(x, z, low, w_dt, dt_bias, a2, skip, state, state_slots, cu_q)
+    out_stride = _gpu_rows(out)
+    T, inner = x.shape
+    N = a2.shape[0]
+    _need(x.dtype == z.dtype == low.dtype == w_dt.dtype == out.dtype, "the activations differ in type")
+    _need(z.shape[0] == low.shape[0] == out.shape[0] == T and z_off >= 0 and z_off + inner <= z.shape[1] and out.shape[1] == inner
+          and low.shape[1] >= rank + 2 * N and tuple(w_dt.shape) == (inner, rank), "selective_scan shapes")
+    for t, n, what in ((dt_bias, inner, "dt_bias"), (a2, N * inner, "a2"), (skip, inner, "skip")):
+        _need(t.dtype == torch.float32 and t.numel() == n, f"{what} must be float32 with {n} elements")
+    _need(state.dtype == torch.float32 and state.dim() >= 2 and state[0].numel() >= N * inner, "the state must be float32 [slots, >= n_state * inner]")
+    _i32(state_slots, n_requests, "state_slots")
+    _i32(cu_q, n_requests + 1, "cu_q")
+    lib = _load("selective_scan")
+    head = (dtype_code(x.dtype), _ptr(x), _ptr(z), z.shape[1], int(z_off), _ptr(low), low.shape[1], _ptr(w_dt), _ptr(dt_bias), _ptr(a2),
+            _ptr(skip), _ptr(state), state[0].numel(), state.shape[0], _ptr(state_slots), _ptr(cu_q), _ptr(out), out_stride, float(out_scale))
+    if segments is None:
+        _need(T == n_requests, "single tokens: one a request")
+        _check(lib.cw_selective_scan_step(*head, n_requests, inner, N, int(rank), _stream()), "selective_scan_step")
+        return out
+    items, n_segments, seg_tokens, first = segments
+    _i32(items, 4 * n_segments, "segments")
+    _i32(first, n_requests + 1, "first segments")
+    workspace = torch.empty(int(lib.cw_selective_scan_workspace_floats(T, n_segments, inner, N)), dtype=torch.float32, device=x.device)
+    _check(lib.cw_selective_scan_segments(*head, _ptr(items), n_segments, int(seg_tokens), _ptr(first), _ptr(workspace), n_requests, T,
+                                          inner, N, int(rank), _stream()), "selective_scan_segments")
+    return out
+
+
+# ---------------------------------------------------------------------------------------------
+def matrix_memory_chunk(dtype, dim: int) -> int:
+    """Tokens of a chunk of ``matrix_memory`` for keys of ``dim`` elements; 0: beyond the kernels."""
+    return int(_load("matrix_memory").cw_matrix_memory_chunk(dtype_code(dtype), dim))
+
+
+def matrix_memory_slot(heads: int, dim: int, vdim: int) -> int:
+    """Floats of a request's slot: the matrices, then two copies of each head's key sum and maximum."""
+    return heads * dim * vdim + 2 * heads * (dim + 1)
+
+
+def matrix_memory(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, x: torch.Tensor, gate_w, gate_b, cap: float, q_scale: float,
+                  state, state_slots, cu_q, ctx_lens, n_requests: int, heads: int, dim: int, vdim: int, chunks=None,
+                  split: int = 1) -> torch.Tensor:
+    """The matrix memory with exponential gates and a running maximum over the step's tokens, from and to each
+    request's slot of ``state`` (float32 [slots, >= matrix_memory_slot]). Columns of ``proj`` hold q, k
+    (heads * dim) and v (heads * vdim); the gates' logarithms are made from the mixer's input ``x`` [T, width]
+    with ``gate_w`` [2 * heads, width] (the input gates' rows, then the forget gates') and ``gate_b`` float32
+    [2 * heads], capped by ``cap`` tanh. Returns every head's output before its norm, float32 [T, heads * vdim].
+
+    ``chunks`` None: every request has one token (``split`` workgroups share a head's columns). Else (items,
+    their number, first chunk of each request)."""
+    _gpu(proj, x, gate_w, gate_b, state, state_slots, cu_q, ctx_lens)
+    T, width = proj.shape
+    _need(x.shape[0] == T and x.dtype == proj.dtype == gate_w.dtype and tuple(gate_w.shape) == (2 * heads, x.shape[1])
+          and gate_b.dtype == torch.float32 and gate_b.numel() == 2 * heads, "the gates take [2 * heads, width] rows and float32 biases")
+    _need(min(q_off, k_off, v_off) >= 0 and max(q_off, k_off) + heads * dim <= width and v_off + heads * vdim <= width, "proj columns")
+    _need(state.dtype == torch.float32 and state.dim() >= 2 and state[0].numel() >= matrix_memory_slot(heads, dim, vdim),
+          "the state must be float32 [slots, matrix_memory_slot]")
+    _step_indices((state_slots, cu_q, ctx_lens), n_requests)
+    y = torch.empty((T, heads * vdim), dtype=torch.float32, device=proj.device)
+    lib = _load("matrix_memory")
+    head = (dtype_code(proj.dtype), _ptr(proj), width, int(q_off), int(k_off), int(v_off), _ptr(x), _ptr(gate_w), _ptr(gate_b), x.shape[1],
+            float(cap), float(q_scale), _ptr(state), state[0].numel(), state.shape[0], _ptr(state_slots), _ptr(cu_q), _ptr(ctx_lens), _ptr(y))
+    if chunks is None:
+        _need(T == n_requests, "single tokens: one a request")
+        _check(lib.cw_matrix_memory_step(*head, n_requests, heads, dim, vdim, int(split), _stream()), "matrix_memory_step")
+        return y
+    items, n_chunks, first = chunks
+    _i32(items, 4 * n_chunks, "chunks")
+    _i32(first, n_requests + 1, "first chunks")
+    workspace = torch.empty(int(lib.cw_matrix_memory_workspace_floats(T, n_requests, n_chunks, heads, dim, vdim)), dtype=torch.float32,
+                            device=proj.device)
+    _check(lib.cw_matrix_memory_chunks(*head, _ptr(items), n_chunks, _ptr(first), _ptr(workspace), n_requests, T, heads, dim, vdim,
+                                       _stream()), "matrix_memory_chunks")
+    return y

@@ -218,3 +218,52 @@ class PostNormBlock(BranchNormBlock):
     that of :class:`BranchNormBlock`; what differs is what its norms do when a branch joins. The
     feed-forward and its norm may be absent."""
 
+
+class SandwichBlock:
+    """x = x + N1b(mixer(N1(x))); x = x + N2b(ffn(N2(x))): a norm before and a norm behind each sublayer
+    (``DynamicTanh`` parts: what joins the stream may be normed in the kernel that norms the stream next).
+    The feed-forward and its two norms may be absent.
+
+    The stream is float32. A branch is handed on un-normed and unadded (``ops.NormedBranch``) to the norm that
+    comes next when that norms it inside its kernel (``accepts_normed_branch``); else the block joins it."""
+
+    def __init__(self, mixer, mixer_norm, mixer_post_norm, feed_forward=None, ffn_norm=None, ffn_post_norm=None) -> None:
+        if len({feed_forward is None, ffn_norm is None, ffn_post_norm is None}) != 1:
+            raise ValueError("a block has a feed-forward and its two norms, or none of them")
+        for norm in (mixer_norm, ffn_norm):
+            if norm is not None and not getattr(norm, "accepts_normed_branch", False):
+                raise TypeError("the norms of a 'sandwich' block norm the branch that joins ahead of them")
+        self.mixer, self.mixer_norm, self.mixer_post_norm = mixer, mixer_norm, mixer_post_norm
+        self.feed_forward, self.ffn_norm, self.ffn_post_norm = feed_forward, ffn_norm, ffn_post_norm
+        for part in (mixer, feed_forward):
+            if hasattr(part, "partial_ok"):
+                part.partial_ok = True
+
+    def parts(self) -> dict:
+        parts = {"mixer": self.mixer}
+        if self.feed_forward is not None:
+            parts["feed_forward"] = self.feed_forward
+        parts.update(mixer_norm=self.mixer_norm, mixer_post_norm=self.mixer_post_norm)
+        if self.feed_forward is not None:
+            parts.update(ffn_norm=self.ffn_norm, ffn_post_norm=self.ffn_post_norm)
+        return parts
+
+    def first_norm(self):
+        return self.mixer_norm
+
+    def forward(self, resid, delta, ctx, cache):
+        last = ops.NormedBranch(self.mixer.forward(self.mixer_norm.forward(resid, delta), ctx, cache), self.mixer_post_norm)
+        if self.feed_forward is not None:
+            last = ops.NormedBranch(self._feed(self.ffn_norm.forward(resid, last), ctx), self.ffn_post_norm)
+        if getattr(ctx, "next_norm_accepts_normed", False):
+            return last
+        last.norm.join(resid, last.branch)
+        return None
+
+    def _feed(self, x, ctx):
+        """The feed-forward's output; a routed one leaves adding its pairs to the norm (but for identity experts,
+        whose row is the feed-forward's input)."""
+        pending = getattr(self.feed_forward, "forward_pairs", None)
+        if pending is not None and not getattr(self.feed_forward.spec, "num_identity", 0):
+            return pending(x, ctx)
+        return self.feed_forward.forward(x, ctx)

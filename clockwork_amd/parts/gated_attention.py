@@ -13,7 +13,9 @@ given back while the request runs.
 bfloat16 steps whose head size the kernels for plain grouped attention are built for run on
 those (the two planes have the layout of a key/value cache); everything else, float32 included,
 on the kernel for paged rows, which is also the one that knows kept first positions behind a
-window and a cap on the scores. The norm may come before or after the rotation and may lack
+window and a cap on the scores. A mixer whose projections pass a short convolution, or whose norm spans
+the whole projection, has a kernel of its own between product and attention (the queries then leave
+the product's rows), and keeps the convolution's latest inputs as a state beside its pages. The norm may come before or after the rotation and may lack
 weights, the rotation may pair halves or neighbours, queries may carry a factor that grows with
 the logarithm of their position, and the gate may be one number a head: all in the same kernels.
 """
@@ -23,18 +25,22 @@ from __future__ import annotations
 import torch
 
 from clockwork_amd import ops
-from clockwork_amd.config.spec import PagedRowsSpec, ParamSpec
+from clockwork_amd.config.spec import CacheNeeds, PagedRowsSpec, ParamSpec, StateSpec
 from clockwork_amd.parts.attention import attention_plan
 from clockwork_amd.parts.base import EntryCache, Part
+from clockwork_amd.parts.rope import rotary_frequencies
 from clockwork_amd.parts.sink_attention import longest_key_range, query_runs
 from clockwork_amd.parts.specs import GatedAttentionSpec, RopePairsSpec
 
 
 class GatedAttention(Part):
     graph_safe = True
+    partial_ok = False   # may the output come as ``ops.PartialSums``? A block whose next norm adds them up sets it
 
     def __init__(self, spec: GatedAttentionSpec) -> None:
         self.spec = spec
+        # the convolution and a norm over the projection share a kernel, which leaves the queries apart
+        self.prepares = bool(spec.conv_taps) or (spec.qk_norm and spec.qk_norm_over == "projection")
         self.q_width = spec.num_heads * spec.key_dim
         self.k_width = spec.num_kv_heads * spec.key_dim
         self.v_width = spec.num_kv_heads * spec.value_dim
@@ -57,14 +63,19 @@ class GatedAttention(Part):
         if s.out_bias:
             specs["out_bias"] = ParamSpec((s.hidden_size,), precision="compute", init=("normal", 0.02))
         if s.qk_norm and s.qk_norm_weight:
-            specs["q_norm"] = ParamSpec((s.key_dim,), precision="stored", init=("one_plus_uniform", 0.3))
-            specs["k_norm"] = ParamSpec((s.key_dim,), precision="stored", init=("one_plus_uniform", 0.3))
+            whole = s.qk_norm_over == "projection"
+            for name, width in (("q_norm", self.q_width), ("k_norm", self.k_width)):
+                specs[name] = ParamSpec((width if whole else s.key_dim,), precision="float32" if whole else "stored",
+                                        init=("one_plus_uniform", 0.3))
+        if s.conv_taps:
+            specs["conv_weight"] = ParamSpec((self.g_off, s.conv_taps), precision="float32", init=("normal", 0.5))
         return specs
 
     def cache_need(self):
         s = self.spec
-        return PagedRowsSpec((("k", (s.num_kv_heads, s.key_dim)), ("v", (s.num_kv_heads, s.value_dim))), window=s.window,
+        rows = PagedRowsSpec((("k", (s.num_kv_heads, s.key_dim)), ("v", (s.num_kv_heads, s.value_dim))), window=s.window,
                              keep_first=s.keep_first)
+        return CacheNeeds((rows, StateSpec((s.conv_taps * self.g_off,), "float32"))) if s.conv_taps else rows
 
     def _plain_kernels(self, dtype) -> bool:
         """Do the kernels for plain grouped attention take these heads? bfloat16, keys and values
@@ -78,7 +89,7 @@ class GatedAttention(Part):
     def kernel_libraries(self) -> list:
         # the library of plain grouped attention is loaded (and, if missing, built) when the part is
         # bound as bfloat16 with a head size it takes: a float32 engine never needs it
-        return [("rowwise", None), ("rows_attention", None)]
+        return [("rowwise", None), ("rows_attention", None)] + ([("short_conv", None)] if self.prepares else [])
 
     def bind(self, params, device, dtype) -> None:
         s = self.spec
@@ -88,12 +99,17 @@ class GatedAttention(Part):
         self.rot_dims = s.position.rotary_dim if s.position is not None else 0
         self.pairing = "neighbours" if isinstance(s.position, RopePairsSpec) else "halves"
         self.norm_order = "none" if not s.qk_norm else ("after" if s.qk_norm_after_rotation else "before")
-        self.freq = None
+        self.freq, self.rot_mult = None, 1.0
         if self.rot_dims:
-            # base^(-2i / n), made on the host in float64 and rounded once
-            freq = torch.tensor([float(s.position.theta) ** (-2.0 * i / self.rot_dims) for i in range(self.rot_dims // 2)],
-                                dtype=torch.float64)
+            freq, self.rot_mult = rotary_frequencies(s.position)
             self.freq = freq.to(torch.float32).to(device)
+        if self.rot_mult != 1.0 and not self.prepares:
+            raise NotImplementedError("a factor on what is rotated goes with a convolution or a norm over the projection")
+        self.conv = params.get("conv_weight")
+        if self.prepares:
+            self.conv_run = ops.qkv_conv_run(self.q_width, self.k_width, self.rot_dims, s.conv_taps)
+            if not self.conv_run:
+                raise ValueError(f"projections of {self.q_width} and {self.k_width} elements with {s.conv_taps} taps are beyond the kernel")
         self.dtype = dtype
         pad = (-self.in_width) % 8
         if pad and dtype == torch.bfloat16:
@@ -136,35 +152,59 @@ class GatedAttention(Part):
 
     def prepare(self, ctx) -> None:
         self._plan(ctx)
+        if self.prepares:
+            query_runs(ctx, self.conv_run)
 
     def forward(self, x: torch.Tensor, ctx, cache: EntryCache) -> torch.Tensor:
-        s = self.spec
         policy = getattr(ctx, "products", None)
-        if not cache.writes:
-            raise NotImplementedError("this mixer writes its own keys and values: it cannot borrow another entry's cache")
-        k_plane, v_plane = cache.planes["k"], cache.planes["v"]
         proj = ops.linear(x, self.in_weight, policy=policy)
-        ops.headnorm_rope_store(proj, 0, self.q_width, self.v_off, s.num_heads, s.num_kv_heads, s.key_dim, self.v_width,
-                                self.in_bias, self.q_norm, self.k_norm, s.norm_eps, ctx.positions, self.freq, self.rot_dims,
-                                ctx.slots[cache.group], k_plane, v_plane, values_from_keys=not self.own_values,
-                                pairing=self.pairing, norm=self.norm_order, query_temperature=s.query_temperature)
         out = torch.empty((x.shape[0], self.out_width), dtype=x.dtype, device=x.device)
+        self.mix(proj, 0, out, x, ctx, cache)
+        return ops.linear(out, self.out_weight, self.out_bias, partial_ok=self.partial_ok, policy=policy)
+
+    def joins(self) -> bool:
+        """May a pair of mixers make this one's products together with the other's (``mix`` with an output scale)?"""
+        return self.prepares and not self.spec.out_bias
+
+    def mix(self, proj: torch.Tensor, off: int, out: torch.Tensor, x, ctx, cache: EntryCache, scale: float = 1.0) -> None:
+        """What stands between the two products: from the columns of ``proj`` that begin at ``off`` (what
+        ``in_weight`` made of the input ``x``) to ``out`` [T, out_width], times ``scale``."""
+        s = self.spec
+        pages = cache.members[0] if s.conv_taps else cache
+        if not pages.writes:
+            raise NotImplementedError("this mixer writes its own keys and values: it cannot borrow another entry's cache")
+        k_plane, v_plane = pages.planes["k"], pages.planes["v"]
+        if self.prepares:
+            items, n_items = query_runs(ctx, self.conv_run)
+            state = cache.members[1].state if s.conv_taps else None
+            # a factor of the output is a factor of the values
+            q = ops.qkv_conv_store(proj, off, self.q_width, self.k_width, self.v_width, s.key_dim, self.conv, state, ctx.state_slots,
+                                   ctx.cu_q, ctx.ctx_lens, items, n_items, ctx.num_requests, self.q_norm, self.k_norm, s.norm_eps,
+                                   ctx.positions, self.freq, self.rot_dims, self.rot_mult, scale, ctx.slots[pages.group], k_plane, v_plane)
+        else:
+            if off or scale != 1.0:
+                raise NotImplementedError("this mixer's queries stay in the first columns of the product's rows")
+            q = proj
+            ops.headnorm_rope_store(proj, 0, self.q_width, self.v_off, s.num_heads, s.num_kv_heads, s.key_dim, self.v_width,
+                                    self.in_bias, self.q_norm, self.k_norm, s.norm_eps, ctx.positions, self.freq, self.rot_dims,
+                                    ctx.slots[pages.group], k_plane, v_plane, values_from_keys=not self.own_values,
+                                    pairing=self.pairing, norm=self.norm_order, query_temperature=s.query_temperature)
+        cache = pages
         if self.plain:
-            self._attend_plain(proj, out, ctx, cache, k_plane, v_plane)
+            self._attend_plain(q, out, ctx, cache, k_plane, v_plane)
         else:
             items, n_items, runs = self._plan(ctx)
-            ops.rows_attention(proj, (proj.shape[1], s.key_dim), out, (out.shape[1], s.value_dim), k_plane, v_plane,
+            ops.rows_attention(q, (q.shape[1], s.key_dim), out, (out.stride(0), s.value_dim), k_plane, v_plane,
                                ctx.block_tables[cache.group], ctx.ctx_lens, ctx.cu_q, items, n_items, s.num_heads, s.num_kv_heads,
                                s.key_dim, s.value_dim, cache.block_size, s.scale, maps=1,
                                mask="window" if s.window is not None else "causal", mask_size=s.window or 0,
                                keep_first=s.keep_first, softcap=s.softcap or 0.0, mfma=self.rows_mfma, key_runs=runs,
-                               head_gate=(proj, self.g_off) if self._gate_inside else None)
+                               head_gate=(proj, off + self.g_off) if self._gate_inside else None)
         if s.output_gate and not (self._gate_inside and not self.plain):
             bias_free = self.in_bias is None
             if not bias_free:
                 raise NotImplementedError("an output gate with a bias")
-            ops.sigmoid_mul_(out, proj, self.g_off, group=s.value_dim if s.gate_per_head else 1)
-        return ops.linear(out, self.out_weight, self.out_bias, policy=policy)
+            ops.sigmoid_mul_(out, proj, off + self.g_off, group=s.value_dim if s.gate_per_head else 1)
 
     def _attend_plain(self, q, out, ctx, cache, k_plane, v_plane) -> None:
         """The kernels of plain grouped attention on the two planes (each [rows, kv_heads, size])."""

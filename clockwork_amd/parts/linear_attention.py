@@ -202,3 +202,79 @@ class ShiftedRecurrence(Part):
         else:
             out = ops.linear_recurrence(*common, *sizes, decay="double_exp_tanh", bonus=self.bonus, decay_input=decay_input)
         return ops.linear(out, self.out_weight, policy=policy)
+
+
+class MatrixMemory(Part):
+    """A matrix memory with exponential gates and a running maximum (``MatrixMemorySpec``).
+
+    One product makes q, k, v and the output gate of every token. A step of single tokens: one kernel
+    a (request, head, part of its columns) makes the gates' logarithms from the mixer's input, moves
+    state and maximum on and reads the output. Any other step: the gates of all tokens, then chunks of
+    tokens side by side (what each adds, the start states carried from chunk to chunk under the running
+    maximum, each chunk's outputs), products on the matrix cores. Then one kernel for the heads' norm
+    and the gate, and the output product. A request's slot is float32: the matrices, then two copies of
+    every head's key sum and maximum, one for even and one for odd positions."""
+
+    graph_safe = True
+    partial_ok = False   # may the output come as ``ops.PartialSums``? A block whose next norm adds them up sets it
+
+    def __init__(self, spec) -> None:
+        self.spec = spec
+        qk, v = spec.num_heads * spec.key_dim, spec.num_heads * spec.value_dim
+        # columns of the input product: q, k, v, gate
+        self.k_off, self.v_off, self.g_off, self.in_width = qk, 2 * qk, 2 * qk + v, 2 * qk + 2 * v
+
+    def param_specs(self):
+        s = self.spec
+        return {
+            "in_weight": ParamSpec((self.in_width, s.hidden_size)),
+            # the input gates' rows, then the forget gates'
+            "gate_weight": ParamSpec((2 * s.num_heads, s.hidden_size), init=("normal", 0.1)),
+            "gate_bias": ParamSpec((2 * s.num_heads,), precision="float32", init=("uniform", -2.0, 4.0)),
+            "norm_weight": ParamSpec((s.num_heads * s.value_dim,), precision="float32", init=("one_plus_uniform", 0.1)),
+            "out_weight": ParamSpec((s.hidden_size, s.num_heads * s.value_dim)),
+        }
+
+    def cache_need(self):
+        s = self.spec
+        return StateSpec((s.num_heads * s.key_dim * s.value_dim + 2 * s.num_heads * (s.key_dim + 1),), "float32")
+
+    def kernel_libraries(self) -> list:
+        return [("matrix_memory", None), ("state_space", None)]
+
+    def bind(self, params, device, dtype) -> None:
+        s = self.spec
+        self.chunk = ops.matrix_memory_chunk(dtype, s.key_dim)
+        if not self.chunk:
+            raise ValueError(f"keys of {s.key_dim} elements a head are beyond the matrix-memory kernels (256)")
+        self.in_weight, self.out_weight = params["in_weight"], params["out_weight"]
+        pad = (-self.in_width) % 8
+        if pad and dtype == torch.bfloat16:
+            # rows of the product that begin at multiples of 16 bytes
+            self.in_weight = torch.cat([self.in_weight, self.in_weight.new_zeros((pad, s.hidden_size))])
+        self.gate_weight, self.gate_bias = params["gate_weight"], params["gate_bias"]
+        self.norm_weight = params["norm_weight"]
+
+    def _chunks(self, ctx):
+        """None for a step of single tokens, else what ``ops.matrix_memory`` takes as ``chunks``."""
+        from clockwork_amd.parts.state_space import request_chunks
+
+        return request_chunks(ctx, self.chunk) if max(ctx.h_q_lens, default=0) > 1 else None
+
+    def prepare(self, ctx) -> None:
+        self._chunks(ctx)
+
+    def shape_class(self, q_lens, ctx_lens):
+        return "chunks" if max(q_lens, default=0) > 1 else "single tokens"
+
+    def forward(self, x: torch.Tensor, ctx, cache: EntryCache):
+        s = self.spec
+        policy = getattr(ctx, "products", None)
+        proj = ops.linear(x, self.in_weight, policy=policy)
+        # single tokens: a head's columns are shared by workgroups while compute units are idle
+        split = min(4, max(1, ctx.num_compute_units // max(1, ctx.num_requests * s.num_heads)))
+        y = ops.matrix_memory(proj, 0, self.k_off, self.v_off, x, self.gate_weight, self.gate_bias, s.gate_cap, s.key_dim ** -0.5,
+                              cache.state, ctx.state_slots, ctx.cu_q, ctx.ctx_lens, ctx.num_requests, s.num_heads, s.key_dim, s.value_dim,
+                              chunks=self._chunks(ctx), split=split)
+        out = ops.gated_parts_norm(y, proj, self.g_off, self.norm_weight, s.norm_eps, s.num_heads, gate_last=True)
+        return ops.linear(out, self.out_weight, partial_ok=self.partial_ok, policy=policy)

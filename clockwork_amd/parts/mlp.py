@@ -38,11 +38,12 @@ class SwiGLU(Part):
 
 
 class GatedMLP(Part):
-    """down(act(gate(x)) * up(x)) with the activation the spec names. "silu" takes the fused
+    """down(act(gate(x)) * up(x)) with the activation the spec names. "silu" and "relu" take the fused
     kernels of :class:`SwiGLU`; "gelu_tanh" runs the gate/up product, one kernel for
     gelu_tanh(gate) * up in float32, and the down product."""
 
     graph_safe = True
+    partial_ok = False   # may the output come as ``ops.PartialSums``? A block whose next norm adds them up sets it
 
     def __init__(self, spec) -> None:
         self.spec = spec
@@ -52,7 +53,7 @@ class GatedMLP(Part):
         return {"gate_up_weight": ParamSpec((2 * I, H)), "down_weight": ParamSpec((H, I))}
 
     def kernel_libraries(self) -> list:
-        return [("rowwise", None)] if self.spec.activation != "silu" else []
+        return [("rowwise", None)] if self.spec.activation == "gelu_tanh" else []
 
     def bind(self, params, device, dtype) -> None:
         self.gate_up = params["gate_up_weight"]
@@ -60,8 +61,9 @@ class GatedMLP(Part):
 
     def forward(self, x, ctx) -> torch.Tensor:
         policy = getattr(ctx, "products", None)
-        if self.spec.activation == "silu":
-            return ops.linear(ops.linear_swiglu(x, self.gate_up, policy=policy), self.down, policy=policy)
+        if self.spec.activation != "gelu_tanh":
+            inner = ops.linear_swiglu(x, self.gate_up, policy=policy, limit=ops.RELU_GATE if self.spec.activation == "relu" else 0.0)
+            return ops.linear(inner, self.down, partial_ok=self.partial_ok, policy=policy)
         gate_up = ops.linear(x, self.gate_up, policy=policy)
         inner = torch.empty((x.shape[0], self.spec.intermediate_size), dtype=x.dtype, device=x.device)
         return ops.linear(ops.gelu_tanh_mul(gate_up, inner), self.down, policy=policy)

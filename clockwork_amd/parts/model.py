@@ -176,7 +176,7 @@ class DecoderModel:
         for i, entry in enumerate(run):
             if entry.reenter is not None:
                 # the stream is made anew from itself (with what is pending) and the model's input
-                if isinstance(delta, (ops.GatedBranches, ops.StreamImage, ops.WithStreamInput)):
+                if isinstance(delta, (ops.GatedBranches, ops.StreamImage, ops.WithStreamInput, ops.NormedBranch)):
                     raise TypeError("the stream is re-entered with plain pending outputs only")
                 resid = self.reentry.forward(resid, delta, again, entry.reenter, ctx)
                 delta = None
@@ -190,6 +190,7 @@ class DecoderModel:
             else:
                 nxt = self.final_norm
             ctx.next_norm_accepts_pending = bool(getattr(nxt, "accepts_pending", False))
+            ctx.next_norm_accepts_normed = bool(getattr(nxt, "accepts_normed_branch", False))
             ctx.next_norm_accepts_gated = bool(getattr(nxt, "accepts_gated", False))
             delta = self.layers[entry.layer].forward(resid, delta, ctx, caches[i])
         if ctx.num_logit_rows == 0:

@@ -11,7 +11,7 @@ the sum over a token's pairs in float32 (not needed when top_k is 1). The expert
 stacked: gate_up [experts, 2 * ff, hidden] (an expert's gate rows, then its up rows) and down
 [experts, hidden, ff]. Cache manager and scheduler are not involved.
 
-Options of the spec: a correction per expert that joins the scores for the choice only; experts
+Options of the spec: a bias per expert on its logit; a correction per expert that joins the scores for the choice only; experts
 in runs of which only the best can be chosen (both inside the router's kernel); a shared expert
 that every token uses (the dense gated products) whose output, times a logistic gate of the same
 input (one more row of the router's product), joins in the kernel that sums a token's pairs; a
@@ -44,6 +44,8 @@ class RoutedExperts(Part):
             "gate_up_weight": ParamSpec((s.num_experts * 2 * s.intermediate_size, s.hidden_size)),
             "down_weight": ParamSpec((s.num_experts * s.hidden_size, s.intermediate_size)),
         }
+        if s.router_bias:
+            specs["router_bias"] = ParamSpec((s.num_choices,), precision="float32", init=("normal", 0.1))
         if s.choice_correction:
             specs["correction"] = ParamSpec((s.num_choices,), precision="float32", init=("normal", 0.1))
         if s.shared_intermediate is not None:
@@ -62,7 +64,7 @@ class RoutedExperts(Part):
         self.router = params["router_weight"]
         self.gate_up = params["gate_up_weight"].view(s.num_experts, 2 * s.intermediate_size, s.hidden_size)
         self.down = params["down_weight"].view(s.num_experts, s.hidden_size, s.intermediate_size)
-        self.correction = params.get("correction")
+        self.router_bias, self.correction = params.get("router_bias"), params.get("correction")
         self.shared_gate_up, self.shared_down = params.get("shared_gate_up_weight"), params.get("shared_down_weight")
         self.kernel = None   # a kernel's name: that one for every step (tests); None: chosen by the step's shape
 
@@ -70,7 +72,7 @@ class RoutedExperts(Part):
         """(choice int32 [T, top_k], score float32 [T, top_k]), and with a gated shared expert
         its gate, float32 [T, 1], as a third."""
         s = self.spec
-        return ops.moe_route(x, self.router, s.top_k, s.router, s.renormalize, correction=self.correction, groups=s.groups,
+        return ops.moe_route(x, self.router, s.top_k, s.router, s.renormalize, bias=self.router_bias, correction=self.correction, groups=s.groups,
                              extra=1 if s.shared_gate else 0, renorm_eps=s.renorm_eps, scale=s.score_scale)
 
     def _shared(self, x, ctx):

@@ -88,6 +88,11 @@ class DynamicTanh(Part):
 
     graph_safe = True
     accepts_stream_input = True
+    # takes a delta that is an ops.NormedBranch: the branch's own Dynamic Tanh, the residual sum and this norm in
+    # one kernel; a branch may be plain, float32 partial sums or a routed feed-forward's pairs
+    accepts_normed_branch = True
+    accepts_partial_sums = True
+    accepts_routed_sum = True
 
     def __init__(self, spec) -> None:
         self.spec = spec
@@ -114,11 +119,24 @@ class DynamicTanh(Part):
         extra = None
         if isinstance(delta, ops.WithStreamInput):
             delta, extra = delta.delta, delta.extra
-        if isinstance(delta, ops.PartialSums):
-            delta = delta.sum(self.dtype)
         n = resid.shape[0] if rows is None else rows.numel()
         out = torch.empty((n, self.spec.size), dtype=self.dtype, device=resid.device)
+        if isinstance(delta, ops.NormedBranch):
+            if extra is None:
+                b = delta.norm
+                return ops.join_dynamic_tanh(resid, delta.branch, b.weight, b.bias, b.alpha, self.weight, self.bias, self.alpha, out, rows)
+            if rows is not None:
+                raise TypeError("a stream input is added before a block, not ahead of chosen rows")
+            delta.norm.join(resid, delta.branch)
+            delta = None
+        if isinstance(delta, ops.PartialSums):
+            delta = delta.sum(self.dtype)
         return ops.add_dynamic_tanh(resid, delta, self.spec.delta_scale, extra, self.weight, self.bias, self.alpha, out, rows)
+
+
+    def join(self, resid: torch.Tensor, branch) -> None:
+        """resid += this norm of ``branch``."""
+        ops.join_dynamic_tanh(resid, branch, self.weight, self.bias, self.alpha)
 
 
 class BranchRMSNorm(Part):

@@ -7,11 +7,30 @@ the rotation itself (model.py:32-35, 92-95) runs in float32 inside the kernel.
 
 from __future__ import annotations
 
+import math
+
 import torch
 
 from clockwork_amd import ops
 from clockwork_amd.parts.base import Part
 from clockwork_amd.parts.specs import RopeNeoxSpec
+
+
+def rotary_frequencies(position) -> tuple:
+    """(frequencies as a float64 tensor [rotary_dim / 2], factor of cosine and sine) of a rotary spec: theta^(-2i /
+    n), through its ``scaling`` if it has one. Made on the host; rounded once, by the caller."""
+    n, theta = position.rotary_dim, float(position.theta)
+    freq = torch.tensor([theta ** (-2.0 * i / n) for i in range(n // 2)], dtype=torch.float64)
+    s = getattr(position, "scaling", None)
+    if s is None:
+        return freq, 1.0
+
+    def dim_of(turns: float) -> float:
+        return n * math.log(s.original / (2.0 * math.pi * turns)) / (2.0 * math.log(theta))
+
+    lo, hi = max(math.floor(dim_of(s.fast)), 0), min(math.ceil(dim_of(s.slow)), n - 1)
+    ramp = ((torch.arange(n // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return freq / s.factor * ramp + freq * (1.0 - ramp), 0.1 * math.log(s.factor) + 1.0
 
 
 class RopeNeox(Part):
@@ -20,6 +39,8 @@ class RopeNeox(Part):
     def __init__(self, spec: RopeNeoxSpec) -> None:
         if spec.rotary_dim % 2:
             raise ValueError(f"rotary_dim {spec.rotary_dim} must be even")
+        if spec.scaling is not None:
+            raise NotImplementedError("this encoding's kernels take unscaled frequencies")
         self.spec = spec
 
     def bind(self, params, device, dtype) -> None:

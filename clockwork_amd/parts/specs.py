@@ -19,15 +19,33 @@ class RMSNormSpec:
 
 
 @dataclass(frozen=True)
+class YarnSpec:
+    """YaRN scaling of rotary frequencies f_i = theta^(-2i / n): with d(t) = n ln(original / (2 pi t)) / (2 ln
+    theta), lo = max(floor(d(fast)), 0), hi = min(ceil(d(slow)), n - 1) and r_i = (i - lo) / max(hi - lo,
+    0.001) cut to [0, 1], f_i becomes f_i (r_i / factor + 1 - r_i); what is rotated is multiplied by
+    0.1 ln(factor) + 1."""
+
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+    def __post_init__(self):
+        if min(self.factor, self.original, self.fast, self.slow) <= 0:
+            raise ValueError("factor, original, fast and slow of a YaRN scaling must be positive")
+
+
+@dataclass(frozen=True)
 class RopeNeoxSpec:
     """Rotary position encoding, half-split pairing (i, i + rotary_dim/2).
 
     inv_freq[j] = 1 / theta^(2j / rotary_dim); the first ``rotary_dim`` elements
-    of each head are rotated, the rest pass through.
+    of each head are rotated, the rest pass through. ``scaling``: a :class:`YarnSpec` or None.
     """
 
     rotary_dim: int
     theta: float
+    scaling: Any = None
 
 
 @dataclass(frozen=True)
@@ -120,7 +138,7 @@ class PositionTableEmbeddingSpec:
 
 @dataclass(frozen=True)
 class GatedMLPSpec:
-    """down(act(gate(x)) * up(x)), no biases; ``activation`` "silu" or "gelu_tanh"
+    """down(act(gate(x)) * up(x)), no biases; ``activation`` "silu", "relu" or "gelu_tanh"
     (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))))."""
 
     hidden_size: int
@@ -128,8 +146,8 @@ class GatedMLPSpec:
     activation: str = "gelu_tanh"
 
     def __post_init__(self):
-        if self.activation not in ("silu", "gelu_tanh"):
-            raise ValueError(f"activation {self.activation!r}: expected 'silu' or 'gelu_tanh'")
+        if self.activation not in ("silu", "relu", "gelu_tanh"):
+            raise ValueError(f"activation {self.activation!r}: expected 'silu', 'relu' or 'gelu_tanh'")
 
 
 @dataclass(frozen=True)
@@ -198,12 +216,18 @@ class DecayedLinearAttentionSpec:
 @dataclass(frozen=True)
 class PairMixerSpec:
     """Two mixers side by side on the same input; the result is the mean of their outputs, each
-    first RMS-normed over the model width with a weight of its own."""
+    first RMS-normed over the model width with a weight of its own, or with ``scales`` (l, r)
+    l * left + r * right, no norms."""
 
     hidden_size: int
     left: Any
     right: Any
-    eps: float
+    eps: float = 1e-6
+    scales: Optional[tuple] = None
+
+    def __post_init__(self):
+        if self.scales is not None and len(self.scales) != 2:
+            raise ValueError(f"scales is (left, right), got {self.scales!r}")
 
 
 @dataclass(frozen=True)
@@ -409,6 +433,51 @@ class StateSpaceSpec:
 
 
 @dataclass(frozen=True)
+class SelectiveScanSpec:
+    """A recurrence whose decay depends on token, channel and state (a selective scan). One product
+    gives a token x and a gate z (``inner`` each); x passes a causal convolution a channel
+    (``conv_taps`` taps, a bias) and silu. A product of x gives a step input of ``dt_rank`` numbers, B
+    and C (``state_dim`` each); d = softplus(W_dt step + bias), one number a channel. Channel c keeps S_c
+    [state_dim] in float32, zero at a request's start: S_cn <- exp(-exp(A_log_cn) d_c) S_cn + d_c x_c B_n,
+    y_c = S_c . C + D_c x_c; y silu(z) is projected back. A request keeps the states and the
+    convolution's latest inputs."""
+
+    hidden_size: int
+    inner: int
+    state_dim: int
+    dt_rank: int
+    conv_taps: int
+
+    def __post_init__(self):
+        if min(self.hidden_size, self.inner, self.state_dim, self.dt_rank, self.conv_taps) < 1:
+            raise ValueError("the sizes of a selective scan must be positive")
+
+
+@dataclass(frozen=True)
+class MatrixMemorySpec:
+    """A matrix memory a head with exponential gates and a running maximum (an mLSTM): q (times
+    key_dim^-1/2), k and v projections; two numbers a token and head, i = c tanh((w_i x + b_i) / c) and
+    f = log logistic(c tanh((w_f x + b_f) / c)) with c = ``gate_cap``. A head keeps S [key_dim, value_dim], n
+    [key_dim] and m in float32, zero at a request's start: m' = max(f + m, i), S <- e^(f + m - m') S +
+    e^(i - m') k v^T, n likewise with k alone, o = S^T q / (max(|n . q|, e^(-m')) + 1e-6). Every head's o is
+    divided by its root mean square (``norm_eps``); the concatenated heads are multiplied by a weight and by
+    the logistic function of one more projection, and projected back."""
+
+    hidden_size: int
+    num_heads: int
+    key_dim: int
+    value_dim: int
+    gate_cap: float
+    norm_eps: float
+
+    def __post_init__(self):
+        if min(self.hidden_size, self.num_heads, self.key_dim, self.value_dim) < 1:
+            raise ValueError("the sizes of a matrix memory must be positive")
+        if not self.gate_cap > 0:
+            raise ValueError(f"gate_cap must be positive, got {self.gate_cap}")
+
+
+@dataclass(frozen=True)
 class GatedAttentionSpec:
     """Grouped softmax attention over paged key rows [kv_heads, key_dim] and value rows
     [kv_heads, value_dim], with options that plain attention has not:
@@ -433,7 +502,12 @@ class GatedAttentionSpec:
     * ``softcap`` c: scores are squashed before the softmax, c * tanh(scale * q . k / c).
     * ``query_temperature`` (coef, every): the query at position p is multiplied by
       1 + coef * ln(floor((p + 1) / every) + 1), after its norm.
-    * ``gate_per_head`` (with ``output_gate``): the gate is one number a head, not one an element."""
+    * ``gate_per_head`` (with ``output_gate``): the gate is one number a head, not one an element.
+    * ``qk_norm_over`` "projection": the norm divides a token's whole query (key) projection by its root
+      mean square and multiplies it by a weight of that size, instead of every head's vector by itself.
+    * ``conv_taps`` n > 0: every channel of the query, key and value projections passes a causal convolution
+      of n taps over the request's tokens (no bias), before norm and rotation; a request also keeps the
+      latest inputs."""
 
     hidden_size: int
     num_heads: int
@@ -455,12 +529,22 @@ class GatedAttentionSpec:
     softcap: Optional[float] = None
     query_temperature: Optional[tuple] = None
     gate_per_head: bool = False
+    qk_norm_over: str = "head"
+    conv_taps: int = 0
 
     def __post_init__(self):
         if self.num_heads < 1 or self.num_kv_heads < 1 or self.num_heads % self.num_kv_heads:
             raise ValueError(f"num_heads {self.num_heads} is not a multiple of num_kv_heads {self.num_kv_heads}")
         if self.key_dim < 1 or self.value_dim < 1:
             raise ValueError("key_dim and value_dim must be positive")
+        if self.qk_norm_over not in ("head", "projection") or self.conv_taps < 0:
+            raise ValueError(f"qk_norm_over {self.qk_norm_over!r}: 'head' or 'projection'; conv_taps {self.conv_taps}: not negative")
+        if self.conv_taps or self.qk_norm_over == "projection":
+            # the kernel that convolves, norms whole projections, rotates and stores has not these options
+            if (self.values != "projection" or self.qkv_bias or self.query_temperature is not None or isinstance(self.position, RopePairsSpec)
+                    or (self.qk_norm and (self.qk_norm_over != "projection" or not self.qk_norm_weight or self.qk_norm_after_rotation))):
+                raise ValueError("a convolution or a norm over the projection goes with projected values, half-split rotation, weighted "
+                                 "norms ahead of it, no biases and no query temperature")
         if self.values not in ("projection", "keys"):
             raise ValueError(f"values {self.values!r}: expected 'projection' or 'keys'")
         if self.values == "keys" and self.value_dim != self.key_dim:
@@ -533,6 +617,8 @@ class RoutedExpertsSpec:
     divides by. ``shared_intermediate`` n: one more expert of inner width n runs for every token
     and its output is added, times logistic(w_sg x) (one number a token) if ``shared_gate``.
 
+    ``router_bias``: a learned float32 number an expert joins its logit.
+
     ``limit`` > 0: an expert is down(g logistic(1.702 g) (u + 1)) with g = min(gate x, limit) and
     u = up x cut to [-limit, limit]; ``shared_limit`` the same for the shared expert. ``score_scale``
     multiplies the chosen scores last. ``num_identity`` n: the router knows n more experts, behind
@@ -555,6 +641,7 @@ class RoutedExpertsSpec:
     shared_limit: float = 0.0
     score_scale: float = 1.0
     num_identity: int = 0
+    router_bias: bool = False
 
     @property
     def num_choices(self) -> int:

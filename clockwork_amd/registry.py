@@ -43,6 +43,7 @@ _BUILTIN_ARCHITECTURES = {
     "Nenodra": "clockwork_amd.models.nenodra",
     "Raranex": "clockwork_amd.models.raranex",
     "Dogudra": "clockwork_amd.models.dogudra",
+    "Tufevik": "clockwork_amd.models.tufevik",
 }
 
 
@@ -114,12 +115,15 @@ _BUILTIN_PARTS = {
     "StreamRMSNormSpec": ("clockwork_amd.parts.norm", "StreamRMSNorm"),
     "PairEmbeddingSpec": ("clockwork_amd.parts.embedding", "PairEmbedding"),
     "StateSpaceSpec": ("clockwork_amd.parts.state_space", "StateSpace"),
+    "SelectiveScanSpec": ("clockwork_amd.parts.state_space", "SelectiveScan"),
+    "MatrixMemorySpec": ("clockwork_amd.parts.linear_attention", "MatrixMemory"),
 }
 _ARRANGEMENTS: dict[str, Callable[..., Any]] = {}
 _BUILTIN_ARRANGEMENTS = {"prenorm": ("clockwork_amd.parts.block", "PreNormBlock"),
                          "parallel": ("clockwork_amd.parts.block", "ParallelBlock"),
                          "branchnorm": ("clockwork_amd.parts.block", "BranchNormBlock"),
                          "postnorm": ("clockwork_amd.parts.block", "PostNormBlock"),
+                         "sandwich": ("clockwork_amd.parts.block", "SandwichBlock"),
                          "twonorm": ("clockwork_amd.parts.block", "TwoNormParallelBlock")}
 
 
