@@ -2,7 +2,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--layers L] [--dtype bfloat16] [--shape 1.5b]
     python bench.py --workload mixed|arrivals|agent [--shape 7b] [--requests 64]
-    python bench.py --design fuvavik|pesorax|nenodra|raranex|dogudra [--size s|m|l] [--layers L] [--batch B]
+    python bench.py --design fuvavik|pesorax|nenodra|raranex|dogudra|tufevik [--size s|m|l] [--layers L] [--batch B]
 
 Default workload: the layer sizes of Qwen2.5-1.5B with random weights (seed 2), bfloat16,
 8 requests that each hold a 2048-token prompt, context limit 4096, pages of 16 tokens. A
@@ -648,9 +648,38 @@ def dogudra_config(size: dict, layers: int, max_positions: int) -> dict:
             "embedding": {"scale": 1.0, "bigram": {"buckets": 65536, "mul_prev": 31, "mul_cur": 7}}, "layers": entries}
 
 
+# Layer sizes for ``--design tufevik``: the same widths and head counts. The parallel mixer has the Qwen2
+# layer's attention heads behind a convolution of four taps, beside a selective scan of twice the model's
+# width with 16 states a channel and a step rank of a sixteenth of the width; the matrix memory has values of
+# the model's width in heads of twice the key size. The first layer's feed-forward is dense; the others
+# route over twelve experts of a quarter of the Qwen2 layer's inner width, four a token (as many active
+# parameters as the dense layer). Layers alternate between the two kinds.
+TUFEVIK_SIZES = {
+    "s": dict(width=896, heads=14, kv_heads=2, dim=64, vdim=64, head_dim=64, memory_heads=7, memory_dim=64, ff=4864, layers=6),
+    "m": dict(width=1536, heads=12, kv_heads=2, dim=128, vdim=128, head_dim=128, memory_heads=6, memory_dim=128, ff=8960, layers=6),
+    "l": dict(width=2048, heads=16, kv_heads=2, dim=128, vdim=128, head_dim=128, memory_heads=8, memory_dim=128, ff=11008, layers=6),
+}
+
+
+def tufevik_config(size: dict, layers: int, max_positions: int) -> dict:
+    routed = {"kind": "moe", "expert": {"ff": size["ff"] // 4}, "router": {"experts": 12, "top": 4}}
+    rot = {"base": 500000.0, "dims": size["dim"], "scaling": {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}}
+    parallel = {"left": {"heads": size["heads"], "kv_heads": size["kv_heads"], "dim": size["dim"], "vdim": size["vdim"], "conv": 4,
+                         "scale": size["dim"] ** -0.5, "rot": rot},
+                "right": {"inner": 2 * size["width"], "state": 16, "conv": 4, "dt_rank": size["width"] // 16},
+                "left_scale": 0.7, "right_scale": 0.7}
+    memory = {"heads": size["memory_heads"], "dim": size["memory_dim"], "vdim": 2 * size["memory_dim"], "gate_cap": 15.0}
+    entries = []
+    for i in range(layers):
+        mlp = {"kind": "dense", "ff": size["ff"]} if i == 0 else routed
+        entries.append({"type": "mlstm", "mixer": memory, "mlp": mlp} if i % 2 else {"type": "parallel", "mixer": parallel, "mlp": mlp})
+    return {"architecture": "Tufevik", "vocab": DESIGN_VOCAB, "width": size["width"], "norm": {"eps": 1e-6},
+            "embedding": {"scale": size["width"] ** 0.5}, "layers": entries}
+
+
 DESIGNS = {"fuvavik": (FUVAVIK_SIZES, fuvavik_config), "pesorax": (PESORAX_SIZES, pesorax_config),
            "nenodra": (NENODRA_SIZES, nenodra_config), "raranex": (RARANEX_SIZES, raranex_config),
-           "dogudra": (DOGUDRA_SIZES, dogudra_config)}
+           "dogudra": (DOGUDRA_SIZES, dogudra_config), "tufevik": (TUFEVIK_SIZES, tufevik_config)}
 
 
 def qwen2_config_like(size: dict, layers: int, max_positions: int) -> dict:

@@ -41,10 +41,18 @@ struct AttnParams {
   float* part_o;          // [n_items, nkv * n_chunks, n_splits, ROWS, HD] unnormalised outputs
   float* part_ml;         // [n_items, nkv * n_chunks, n_splits, ROWS, 2] running max, sum
   const void* zeros;      // at least HD zero elements: what a masked key or value row is loaded from
+  const void* gate;       // bfloat16 rows, or null: head h's output is multiplied by logistic(gate[token, gate_off + h])
+  int64_t gate_stride;    //   (the matrix-core kernels)
+  int gate_off;
   // decode kernel only
   int identity;           // 1: item i is request i and its one token is row i of the batch (items, cu_q unread)
   int split_keys;         // > 0: split s takes keys [s * split_keys, (s + 1) * split_keys), a multiple of 32
 };
+
+// the factor of a head's output of the token in row ``token`` of the batch
+__device__ __forceinline__ float attn_head_gate(const AttnParams& p, int64_t token, int head) {
+  return p.gate ? cw_logistic(cw_to_float(((const bf16_t*)p.gate)[token * p.gate_stride + p.gate_off + head])) : 1.0f;
+}
 
 // page of a position and the offset inside it; POW2: the page size is a power of two (shift given)
 template <bool POW2> __device__ __forceinline__ int cw_page_index(int pos, int bs, int shift) {
@@ -630,7 +638,7 @@ __global__ __launch_bounds__(256) void attn_decode_bf16_kernel(AttnParams p) {
     }
     if (p.n_splits == 1) {
       ((bf16_t*)p.out)[(int64_t)(q_begin + tok0) * p.out_stride + (kvh * group + hg) * HD + d] =
-          __float2bfloat16(O / L);
+          __float2bfloat16(O / L * attn_head_gate(p, q_begin + tok0, kvh * group + hg));
     } else {
       p.part_o[(base * gh + g) * HD + d] = O;
       if (d == 0) {
@@ -662,6 +670,7 @@ __global__ __launch_bounds__(1024) void attn_decode_merge_kernel(AttnParams p) {
   const int tok0 = ident ? 0 : p.items[4 * item + 1];
   const int q_begin = ident ? item : p.cu_q[p.items[4 * item]];
   const int64_t base = ((int64_t)item * (p.nkv * p.n_chunks) + y) * p.n_splits;
+  const float gate = attn_head_gate(p, q_begin + tok0, kvh * group + hg);
   const int G = blockDim.x / HD;
   const int tg = threadIdx.x / HD, d = threadIdx.x - tg * HD;
   // the thread's first eight partial outputs are requested together with the statistics: they do
@@ -709,7 +718,7 @@ __global__ __launch_bounds__(1024) void attn_decode_merge_kernel(AttnParams p) {
       L += l_s[w];
     }
   }
-  ((bf16_t*)p.out)[(int64_t)(q_begin + tok0) * p.out_stride + (kvh * group + hg) * HD + d] = __float2bfloat16(O / L);
+  ((bf16_t*)p.out)[(int64_t)(q_begin + tok0) * p.out_stride + (kvh * group + hg) * HD + d] = __float2bfloat16(O / L * gate);
 }
 
 #if CW_HD % 32 == 0
@@ -778,7 +787,8 @@ CW_EXPORT int cw_attention_decode_bf16(const void* q, int64_t q_stride, void* ou
                                        const int* items, int n_items, int nh, int nkv, int block_size,
                                        int n_splits, int window, float scale, float* workspace,
                                        int64_t workspace_floats, const void* zeros, int identity,
-                                       int split_keys, int max_ctx, float softcap, hipStream_t stream) {
+                                       int split_keys, int max_ctx, float softcap, const void* gate, int64_t gate_stride,
+                                       int gate_off, hipStream_t stream) {
 #if CW_HAS_DECODE
   if (n_items < 0 || nh <= 0 || nkv <= 0 || nh % nkv != 0 || block_size <= 0 || table_stride <= 0)
     return CW_ERR_ARG;
@@ -797,6 +807,8 @@ CW_EXPORT int cw_attention_decode_bf16(const void* q, int64_t q_stride, void* ou
   p.table_stride = table_stride; p.ctx_lens = ctx_lens; p.cu_q = cu_q; p.items = items;
   p.nh = nh; p.nkv = nkv; p.block_size = block_size; p.bs_shift = cw_log2_or_minus1(block_size);
   p.identity = identity ? 1 : 0; p.split_keys = split_keys;
+  if (gate && (gate_off < 0 || gate_off + nh > gate_stride)) return CW_ERR_ARG;
+  p.gate = gate; p.gate_stride = gate_stride; p.gate_off = gate_off;
   p.gh = cw_attention_decode_gh(group);
   p.n_chunks = (group + p.gh - 1) / p.gh; p.n_splits = n_splits; p.window = window; p.scale = scale; p.softcap = softcap;
   if ((int64_t)nkv * p.n_chunks * p.gh > 65535) return CW_ERR_SIZE;
@@ -1230,7 +1242,7 @@ __global__ __launch_bounds__((PrefillTile<HD, RB>::NT), (HD <= 128 ? 2 : 1)) voi
     float l = l_run[b];
     l = cw_quad_sum(l);
     if (row_pos[b] < 0) continue;
-    const float inv = 1.0f / l;
+    const float inv = attn_head_gate(p, q_begin + (row_pos[b] - (ctx - qlen)), (int)(row_off[b] / HD)) / l;
     bf16_t* orow = (bf16_t*)p.out + (int64_t)(q_begin + (row_pos[b] - (ctx - qlen))) * p.out_stride + row_off[b];
 #pragma unroll
     for (int db = 0; db < ND; ++db) {
@@ -1309,7 +1321,7 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(AttnParams p) {
         for (int sl = 1; sl < slices; ++sl) acc += *reinterpret_cast<const f32x4_t*>(&red[(sl * n_pairs + pair) * 4]);
     }
     if (valid && slice == 0) {
-      const float inv = 1.0f / l;
+      const float inv = attn_head_gate(p, q_begin + tok0 + tokw, kvh * group + hig) / l;
       bf16_t* orow = (bf16_t*)p.out + (int64_t)(q_begin + tok0 + tokw) * p.out_stride + (int64_t)(kvh * group + hig) * HD;
       uint2 two;
       two.x = (uint32_t)cw_float_to_bf16_bits(acc[0] * inv) | ((uint32_t)cw_float_to_bf16_bits(acc[1] * inv) << 16);
@@ -1380,7 +1392,8 @@ CW_EXPORT int cw_attention_prefill_bf16(const void* q, int64_t q_stride, void* o
                                         const int* items, int n_items, int nh, int nkv, int block_size,
                                         int window, float scale, const void* zeros, int row_blocks,
                                         int with_parts, float* workspace, int64_t workspace_floats,
-                                        float softcap, hipStream_t stream) {
+                                        float softcap, const void* gate, int64_t gate_stride, int gate_off,
+                                        hipStream_t stream) {
 #if CW_HAS_PREFILL
   if (zeros == nullptr || ((uintptr_t)zeros & 15)) return CW_ERR_ARG;
   if (n_items < 0 || nh <= 0 || nkv <= 0 || nh % nkv != 0 || block_size <= 0 || table_stride <= 0 || window < 0)
@@ -1398,6 +1411,8 @@ CW_EXPORT int cw_attention_prefill_bf16(const void* q, int64_t q_stride, void* o
   p.nh = nh; p.nkv = nkv; p.block_size = block_size; p.bs_shift = cw_log2_or_minus1(block_size); p.gh = group < 32 ? group : 32;
   p.n_chunks = (group + p.gh - 1) / p.gh; p.n_splits = 1; p.window = window; p.scale = scale; p.softcap = softcap;
   p.part_o = nullptr; p.part_ml = nullptr; p.zeros = zeros;
+  if (gate && (gate_off < 0 || gate_off + nh > gate_stride)) return CW_ERR_ARG;
+  p.gate = gate; p.gate_stride = gate_stride; p.gate_off = gate_off;
   if ((int64_t)nkv * p.n_chunks > 65535) return CW_ERR_SIZE;
   if (with_parts) {
     const int64_t need = cw_attention_prefill_workspace_floats(n_items, nh, nkv, row_blocks);

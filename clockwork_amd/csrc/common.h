@@ -77,6 +77,16 @@ __device__ __forceinline__ float cw_gelu_tanh(float z) {
 __device__ __forceinline__ float cw_silu(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float cw_logistic(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float cw_softplus(float z) { return z > 0.0f ? z + log1pf(expf(-z)) : log1pf(expf(z)); }
+// The same from the bare exp2 and log2 instructions: max(z, 0) + ln(1 + e), e = exp(-|z|). ln(1 + e) is a
+// short power series for small e, where 1 + e would lose its digits, and else ln(u) e / (u - 1) with u = 1 + e
+// as rounded, which takes back what the rounding of the sum took.
+__device__ __forceinline__ float cw_softplus_quick(float z) {
+  const float e = __builtin_amdgcn_exp2f(-1.44269504f * fabsf(z));
+  const float u = 1.0f + e;
+  const float series = e * (1.0f + e * (-0.5f + e * (0.333333333f + e * (-0.25f + e * (0.2f - e * 0.166666667f)))));
+  const float direct = 0.693147181f * __builtin_amdgcn_logf(u) * e * __builtin_amdgcn_rcpf(u - 1.0f);
+  return fmaxf(z, 0.0f) + (e < 0.06f ? series : direct);
+}
 
 template <typename T, int V> struct CwVec;   // V neighbouring elements as float32
 template <typename T> struct CwVec<T, 1> {

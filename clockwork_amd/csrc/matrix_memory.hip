@@ -62,7 +62,7 @@ struct MmParams {
 };
 
 __device__ __forceinline__ float mm_log_input(float z, float cap) { return cap * tanhf(z / cap); }
-__device__ __forceinline__ float mm_log_forget(float z, float cap) { return -cw_softplus(-(cap * tanhf(z / cap))); }
+__device__ __forceinline__ float mm_log_forget(float z, float cap) { return -cw_softplus_quick(-(cap * tanhf(z / cap))); }
 __host__ __device__ inline int mm_round(int n, int to) { return (n + to - 1) / to * to; }
 // n and m of a head as the token at position ``pos`` leaves them
 __device__ __forceinline__ float* mm_norm_at(const MmParams& p, float* slot, int pos, int h) {
@@ -70,11 +70,12 @@ __device__ __forceinline__ float* mm_norm_at(const MmParams& p, float* slot, int
 }
 
 // ---------------------------------------------------------------- gates
-// 16 tokens x 64 gate rows a workgroup, K shared among the four waves, whose sums meet in LDS. The matrix is
+// 16 tokens x 64 gate rows a workgroup, K shared among the eight waves, whose sums meet in LDS. The matrix is
 // the first operand: a lane ends with 4 neighbouring gates of one token.
+#define MM_GATE_WAVES 8
 template <typename T>
-__global__ __launch_bounds__(256) void mm_gate_kernel(MmParams p, int vec) {
-  __shared__ f32x4_t red[4][4][64];
+__global__ __launch_bounds__(MM_GATE_WAVES * 64) void mm_gate_kernel(MmParams p, int vec) {
+  __shared__ f32x4_t red[MM_GATE_WAVES][4][64];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, i = lane & 15, kq = lane >> 4;
   const int t0 = blockIdx.x * 16, g0 = blockIdx.y * 64, G = 2 * p.heads;
   const T* x = (const T*)p.h + (int64_t)min(t0 + i, p.n_tokens - 1) * p.width;
@@ -87,8 +88,8 @@ __global__ __launch_bounds__(256) void mm_gate_kernel(MmParams p, int vec) {
   }
   const int tiles = min(4, (G - g0 + 15) / 16);
   if constexpr (sizeof(T) == 2) {
-#pragma unroll 2
-    for (int k = wave * 32; k < p.width; k += 128) {
+#pragma unroll 4
+    for (int k = wave * 32; k < p.width; k += MM_GATE_WAVES * 32) {
       const int kk = k + kq * 8;
       union { u32x4_t u; bf16x8_t v; uint16_t s[8]; } a, b[4];
       a.u = (u32x4_t){0u, 0u, 0u, 0u};
@@ -114,7 +115,7 @@ __global__ __launch_bounds__(256) void mm_gate_kernel(MmParams p, int vec) {
         if (j < tiles) acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(b[j].v, a.v, acc[j], 0, 0, 0);
     }
   } else {
-    for (int k = wave * 4; k < p.width; k += 16) {
+    for (int k = wave * 4; k < p.width; k += MM_GATE_WAVES * 4) {
       const bool in = k + kq < p.width;
       const float a = in ? cw_to_float(x[k + kq]) : 0.0f;
 #pragma unroll
@@ -127,7 +128,9 @@ __global__ __launch_bounds__(256) void mm_gate_kernel(MmParams p, int vec) {
   __syncthreads();
   const int j = wave;   // a wave finishes one tile
   if (j >= tiles || t0 + i >= p.n_tokens) return;
-  const f32x4_t sum = (red[0][j][lane] + red[1][j][lane]) + (red[2][j][lane] + red[3][j][lane]);
+  f32x4_t sum = red[0][j][lane];
+#pragma unroll
+  for (int v = 1; v < MM_GATE_WAVES; ++v) sum += red[v][j][lane];
 #pragma unroll
   for (int e = 0; e < 4; ++e) {
     const int g = g0 + j * 16 + kq * 4 + e;
@@ -142,16 +145,25 @@ __global__ __launch_bounds__(256) void mm_gate_kernel(MmParams p, int vec) {
 template <typename T> struct MmPad { static constexpr int V = sizeof(T) == 2 ? 8 : 4; };
 
 // Rows of an operand in LDS: ``width`` elements, zeros past the operand's ``n`` and past the ``nt`` tokens.
+// Loads are never conditional (a clamped address, zeros chosen afterwards), so several are on their way at once.
 template <typename T, int THREADS>
 __device__ __forceinline__ void mm_stage(T* dst, int dst_stride, int width, const T* src, int64_t src_stride, int n, int nt, int rows, bool vec) {
   constexpr int V = MmPad<T>::V;
   if (vec) {
-    const int per = width / V;
-    for (int i = threadIdx.x; i < rows * per; i += THREADS) {
-      const int t = i / per, e = (i - t * per) * V;
-      u32x4_t v = (u32x4_t){0u, 0u, 0u, 0u};
-      if (t < nt && e < n) v = *reinterpret_cast<const u32x4_t*>(src + (int64_t)t * src_stride + e);
-      *reinterpret_cast<u32x4_t*>(dst + t * dst_stride + e) = v;
+    const int per = width / V, total = rows * per;
+#pragma unroll 1
+    for (int i0 = threadIdx.x; i0 < total; i0 += 4 * THREADS) {
+      u32x4_t v[4];
+      int at[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int i = min(i0 + u * THREADS, total - 1), t = i / per, e = (i - t * per) * V;
+        at[u] = t * dst_stride + e;
+        const u32x4_t got = *reinterpret_cast<const u32x4_t*>(src + (int64_t)min(t, nt - 1) * src_stride + min(e, n - V));
+        v[u] = (t < nt && e < n) ? got : (u32x4_t){0u, 0u, 0u, 0u};
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u) *reinterpret_cast<u32x4_t*>(dst + at[u]) = v[u];
     }
   } else {
     for (int i = threadIdx.x; i < rows * width; i += THREADS) {
@@ -287,17 +299,18 @@ __global__ __launch_bounds__(256) void mm_carry_kernel(MmParams p) {
   float* st = slot_state + h * DV + e;
   float S[N];
   CwVec<float, N>::load(st, S);
-  for (int c0 = begin; c0 < end; c0 += 4) {
-    float add[4][N], f[4], most[4];   // four chunks' loads side by side
+  constexpr int U = 8;   // chunks whose loads are on their way at once
+  for (int c0 = begin; c0 < end; c0 += U) {
+    float add[U][N], f[U], most[U];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
+    for (int u = 0; u < U; ++u) {
       const int c = min(c0 + u, end - 1);
       CwVec<float, N>::load(p.added + ((int64_t)c * p.heads + h) * DV + e, add[u]);
       f[u] = p.chunk_f[(int64_t)c * p.heads + h];
       most[u] = p.added_n[((int64_t)c * p.heads + h) * (p.D + 1) + p.D];
     }
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
+    for (int u = 0; u < U; ++u) {
       if (c0 + u < end) {
         CwVec<float, N>::store(p.added + ((int64_t)(c0 + u) * p.heads + h) * DV + e, S);
         const float next = fmaxf(m + f[u], most[u]);
@@ -375,11 +388,20 @@ __global__ __launch_bounds__(Q * 4) void mm_chunk_out_kernel(MmParams p, int vec
   mm_stage<T, THREADS>(Vs, SV, Vp, rows + p.v_off + h * p.V + v0, p.stride, V, nt, Q, vec);
   // the start state's columns (a row of it is p.V floats)
   if (!((p.V | V) & 3)) {
-    for (int i = threadIdx.x; i < NK * (MM_COLS / 4); i += THREADS) {
-      const int d = i / (MM_COLS / 4), c = (i - d * (MM_COLS / 4)) * 4;
-      f32x4_t v = (f32x4_t){0.0f, 0.0f, 0.0f, 0.0f};
-      if (d < D && c < V) v = *reinterpret_cast<const f32x4_t*>(start + (int64_t)d * p.V + c);
-      *reinterpret_cast<f32x4_t*>(Ss + d * SS + c) = v;
+#pragma unroll 1
+    for (int i0 = threadIdx.x; i0 < NK * (MM_COLS / 4); i0 += 8 * THREADS) {
+      f32x4_t v[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const int i = i0 + u * THREADS, d = i / (MM_COLS / 4), c = (i - d * (MM_COLS / 4)) * 4;
+        const f32x4_t got = *reinterpret_cast<const f32x4_t*>(start + (int64_t)min(d, D - 1) * p.V + min(c, V - 4));
+        v[u] = (d < D && c < V) ? got : (f32x4_t){0.0f, 0.0f, 0.0f, 0.0f};
+      }
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const int i = i0 + u * THREADS, d = i / (MM_COLS / 4), c = (i - d * (MM_COLS / 4)) * 4;
+        if (d < NK) *reinterpret_cast<f32x4_t*>(Ss + d * SS + c) = v[u];
+      }
     }
   } else {
     for (int i = threadIdx.x; i < NK * MM_COLS; i += THREADS) {
@@ -686,11 +708,24 @@ CW_EXPORT int cw_matrix_memory_chunks(int dtype, const void* proj, int64_t strid
   const bool n4 = ((int64_t)D * V) % 4 == 0 && state_stride % 4 == 0 && !(((uintptr_t)state | (uintptr_t)workspace) & 15);
   const size_t lds_a = mm_state_lds(elem, Q, D), lds_c = mm_out_lds(elem, Q, D);
   const dim3 gate_grid((n_tokens + 15) / 16, (2 * heads + 63) / 64), grid(n_chunks, heads, (V + MM_COLS - 1) / MM_COLS), block(Q * 4);
-  const int64_t per = n4 ? 1024 : 256;
+  // four elements a thread where there are threads enough without
+  const bool n4_pays = n4 && (int64_t)n_requests * heads * D * V >= (int64_t)1024 * 1024;
+  const int64_t per = n4_pays ? 1024 : 256;
   const dim3 carry_grid(n_requests, heads, (unsigned)(((int64_t)D * V + per - 1) / per) + 1);
   const int gate_vec = mm_rows16(dtype, h, gate_w, width);
-#define CW_RAISE(F_, LDS_)                                                                                                      if ((LDS_) > 48 * 1024 && hipFuncSetAttribute((const void*)F_, hipFuncAttributeMaxDynamicSharedMemorySize, (int)(LDS_)) != hipSuccess)     return CW_ERR_LAUNCH
-#define CW_CHUNKS(T_, Q_)                                                                                do {                                                                                                     CW_RAISE((mm_chunk_state_kernel<T_, Q_>), lds_a);                                                      CW_RAISE((mm_chunk_out_kernel<T_, Q_>), lds_c);                                                        hipLaunchKernelGGL((mm_gate_kernel<T_>), gate_grid, dim3(256), 0, stream, p, gate_vec);                hipLaunchKernelGGL((mm_chunk_state_kernel<T_, Q_>), grid, block, lds_a, stream, p, vec);               if (n4) hipLaunchKernelGGL((mm_carry_kernel<4>), carry_grid, dim3(256), 0, stream, p);                 else hipLaunchKernelGGL((mm_carry_kernel<1>), carry_grid, dim3(256), 0, stream, p);                    hipLaunchKernelGGL((mm_chunk_out_kernel<T_, Q_>), grid, block, lds_c, stream, p, vec);               } while (0)
+#define CW_RAISE(F_, LDS_)                                                                                                               \
+  if ((LDS_) > 48 * 1024 && hipFuncSetAttribute((const void*)F_, hipFuncAttributeMaxDynamicSharedMemorySize, (int)(LDS_)) != hipSuccess) \
+    return CW_ERR_LAUNCH
+#define CW_CHUNKS(T_, Q_)                                                                                  \
+  do {                                                                                                     \
+    CW_RAISE((mm_chunk_state_kernel<T_, Q_>), lds_a);                                                      \
+    CW_RAISE((mm_chunk_out_kernel<T_, Q_>), lds_c);                                                        \
+    hipLaunchKernelGGL((mm_gate_kernel<T_>), gate_grid, dim3(MM_GATE_WAVES * 64), 0, stream, p, gate_vec); \
+    hipLaunchKernelGGL((mm_chunk_state_kernel<T_, Q_>), grid, block, lds_a, stream, p, vec);               \
+    if (n4_pays) hipLaunchKernelGGL((mm_carry_kernel<4>), carry_grid, dim3(256), 0, stream, p);            \
+    else hipLaunchKernelGGL((mm_carry_kernel<1>), carry_grid, dim3(256), 0, stream, p);                    \
+    hipLaunchKernelGGL((mm_chunk_out_kernel<T_, Q_>), grid, block, lds_c, stream, p, vec);                 \
+  } while (0)
   if (dtype == CW_F32) { if (Q == 64) CW_CHUNKS(float, 64); else if (Q == 32) CW_CHUNKS(float, 32); else CW_CHUNKS(float, 16); }
   else { if (Q == 64) CW_CHUNKS(bf16_t, 64); else if (Q == 32) CW_CHUNKS(bf16_t, 32); else CW_CHUNKS(bf16_t, 16); }
 #undef CW_CHUNKS

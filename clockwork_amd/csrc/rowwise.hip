@@ -1161,7 +1161,7 @@ CW_EXPORT int cw_stream_beside_input(float* resid, const void* a, const void* b,
 //   * a tensor [T, H] of the activation type,
 //   * ``n_parts`` float32 planes [T, H] whose sum is the branch (a product split over K),
 //   * a routed feed-forward's pairs: the sum over k < top of y[t * top + k, :], or for a choice from
-//     ``experts`` on (an identity expert) of score * resid[t, :], then ``always[t, :]`` (or nullptr).
+//     ``experts`` on (an identity expert; choice == nullptr: none) of score * resid[t, :], then ``always[t, :]`` (or nullptr).
 // float32 inside.
 template <typename T>
 struct PostBranch {
@@ -1177,16 +1177,33 @@ struct PostBranch {
   __device__ __forceinline__ void add(float (&v)[N], const float (&x)[N], int64_t t, int64_t plane, int j, int H) const {
     float b[N];
     if (parts) {
-      for (int p = 0; p < n_parts; ++p) {
-        load(parts + p * plane + t * H + j, b);
+      for (int p = 0; p < n_parts; p += 4) {   // four planes' loads side by side, added in order
+        float q[4][N];
 #pragma unroll
-        for (int i = 0; i < N; ++i) v[i] += b[i];
+        for (int u = 0; u < 4; ++u) load(parts + min(p + u, n_parts - 1) * plane + t * H + j, q[u]);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (p + u < n_parts)
+#pragma unroll
+            for (int i = 0; i < N; ++i) v[i] += q[u][i];
       }
     } else if (pairs) {
       float sum[N];
 #pragma unroll
       for (int i = 0; i < N; ++i) sum[i] = 0.0f;
-      for (int k = 0; k < top; ++k) {
+      if (!choice) {   // no identity experts: every pair has a row
+        for (int k = 0; k < top; k += 4) {
+          float q[4][N];
+#pragma unroll
+          for (int u = 0; u < 4; ++u) load(pairs + (t * top + min(k + u, top - 1)) * H + j, q[u]);
+#pragma unroll
+          for (int u = 0; u < 4; ++u)
+            if (k + u < top)
+#pragma unroll
+              for (int i = 0; i < N; ++i) sum[i] += q[u][i];
+        }
+      }
+      for (int k = 0; choice && k < top; ++k) {
         const int64_t pair = t * top + k;
         if (choice[pair] >= experts) {
           const float f = score[pair];
@@ -1362,14 +1379,14 @@ __global__ __launch_bounds__(256) void join_dyt_kernel(float* __restrict__ resid
   }
 }
 
-CW_EXPORT int cw_join_dyt(float* resid, const void* branch, const float* parts, int n_parts, const void* pairs, const int* choice,
-                          const float* score, const void* always, int top, int experts, const void* bw, const void* bb,
+CW_EXPORT int cw_join_dyt(float* resid, const void* branch, const float* parts, int n_parts, const void* pairs,
+                          const void* always, int top, const void* bw, const void* bb,
                           const float* balpha, const void* w, const void* b, const float* alpha, int w_dtype, void* out, int dtype,
                           const int* rows, int n, int T, int H, hipStream_t stream) {
   if (T < 0 || n < 0 || H <= 0 || !resid || !bw || !balpha || (out && (!w || !alpha)) || (rows && !out)) return CW_ERR_ARG;
   if ((branch != nullptr) + (parts != nullptr) + (pairs != nullptr) != 1) return CW_ERR_ARG;
   if (parts && n_parts < 1) return CW_ERR_ARG;
-  if (pairs && (!choice || !score || top < 1 || experts < 0)) return CW_ERR_ARG;
+  if (pairs && top < 1) return CW_ERR_ARG;
   if (n == 0) return CW_OK;
   const int align = dtype == CW_BF16 ? 8 : 16;
   const bool vec = H % 4 == 0 && !(((uintptr_t)resid | (uintptr_t)parts) & 15) &&
@@ -1379,7 +1396,7 @@ CW_EXPORT int cw_join_dyt(float* resid, const void* branch, const float* parts, 
   const dim3 grid(n, n <= 64 ? (H + per - 1) / per : 1), block(256);
 #define CW_LAUNCH(T_, WT_)                                                                                              \
   do {                                                                                                                  \
-    PostBranch<T_> br{(const T_*)branch, parts, n_parts, (const T_*)pairs, choice, score, (const T_*)always, top, experts}; \
+    PostBranch<T_> br{(const T_*)branch, parts, n_parts, (const T_*)pairs, nullptr, nullptr, (const T_*)always, top, 0}; \
     if (vec)                                                                                                            \
       hipLaunchKernelGGL((join_dyt_kernel<T_, WT_, 4>), grid, block, 0, stream, resid, br, (const WT_*)bw, (const WT_*)bb, balpha, \
                          (const WT_*)w, (const WT_*)b, alpha, (T_*)out, rows, (int64_t)T * H, H);                       \

@@ -112,7 +112,7 @@ __global__ __launch_bounds__(256) void ssc_dt_kernel(SscParams p, int vec) {
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int c = c0 + j * 16 + kq * 4 + e;
-      if (c < p.inner) acc[j][e] = cw_softplus(acc[j][e] + p.dt_bias[c]);
+      if (c < p.inner) acc[j][e] = cw_softplus_quick(acc[j][e] + p.dt_bias[c]);
     }
     const int c = c0 + j * 16 + kq * 4;
     if (!(p.inner & 3)) {
@@ -264,12 +264,15 @@ __global__ __launch_bounds__(256) void ssc_step_kernel(SscParams p, int vec) {
   const int cc = live ? c : p.inner - 1;
   float* st = p.state + slot * p.state_stride + cc;
   // the state's rows are asked for before the step's product is made
-  float ahead[SSC_STEP_AHEAD];
+  float ahead[SSC_STEP_AHEAD], rate[SSC_STEP_AHEAD];
 #pragma unroll
   for (int i = 0; i < SSC_STEP_AHEAD; ++i) {
-    const int n = wave + 4 * i;
-    ahead[i] = n < p.N ? st[(int64_t)n * p.inner] : 0.0f;
+    const int n = min(wave + 4 * i, p.N - 1);
+    ahead[i] = st[(int64_t)n * p.inner];
+    rate[i] = p.a2[(int64_t)n * p.inner + cc];
   }
+  const float bias = p.dt_bias[cc], skip = p.skip[cc];
+  const T z = ((const T*)p.z)[row * p.z_stride + p.z_off + cc];
   const T* pr = (const T*)p.p + row * p.p_stride;
   const float x = cw_to_float(((const T*)p.x)[row * p.inner + cc]);
   for (int i = threadIdx.x; i < 2 * p.N; i += 256) bc[i] = cw_to_float(pr[p.rank + i]);
@@ -295,14 +298,14 @@ __global__ __launch_bounds__(256) void ssc_step_kernel(SscParams p, int vec) {
   }
   red[wave][lane] = s;
   __syncthreads();
-  const float d = cw_softplus((red[0][lane] + red[1][lane]) + (red[2][lane] + red[3][lane]) + p.dt_bias[cc]);
+  const float d = cw_softplus_quick((red[0][lane] + red[1][lane]) + (red[2][lane] + red[3][lane]) + bias);
   const float dx = d * x;
   float acc = 0.0f;
 #pragma unroll
   for (int i = 0; i < SSC_STEP_AHEAD; ++i) {
     const int n = wave + 4 * i;
     if (n < p.N) {
-      const float S = ssc_exp2(d * p.a2[(int64_t)n * p.inner + cc]) * ahead[i] + dx * bc[n];
+      const float S = ssc_exp2(d * rate[i]) * ahead[i] + dx * bc[n];
       if (live) st[(int64_t)n * p.inner] = S;
       acc += S * bc[p.N + n];
     }
@@ -316,9 +319,8 @@ __global__ __launch_bounds__(256) void ssc_step_kernel(SscParams p, int vec) {
   red[wave][lane] = acc;
   __syncthreads();
   if (wave == 0 && live) {
-    const float y = (red[0][lane] + red[1][lane]) + (red[2][lane] + red[3][lane]) + p.skip[c] * x;
-    const float z = cw_to_float(((const T*)p.z)[row * p.z_stride + p.z_off + c]);
-    ((T*)p.out)[row * p.out_stride + c] = cw_from_float<T>(y * cw_silu(z) * p.out_scale);
+    const float y = (red[0][lane] + red[1][lane]) + (red[2][lane] + red[3][lane]) + skip * x;
+    ((T*)p.out)[row * p.out_stride + c] = cw_from_float<T>(y * cw_silu(cw_to_float(z)) * p.out_scale);
   }
 }
 

@@ -10,6 +10,7 @@
 
 #define SHORT_CONV_TOKENS 16                       // tokens of a work item
 #define SHORT_CONV_MAX_TAPS (SHORT_CONV_TOKENS + 1)
+#define SHORT_CONV_RUN 8                           // tokens of a workgroup in the unrolled form (at least its taps - 1)
 
 struct ShortConv {
   const void* in;          // [T, in_stride], the channels from column in_off
@@ -37,10 +38,18 @@ struct ShortConv {
 template <typename T, int V, int TAPS>
 __global__ __launch_bounds__(256) void short_conv_kernel(ShortConv p) {
   const int* item = p.items + 4 * (int64_t)blockIdx.x;
-  const int req = item[0], tok0 = item[1];
+  const int req = item[0];
+  int tok0 = item[1];
   const int row0 = p.cu_q[req], q_len = p.cu_q[req + 1] - row0;
   if (tok0 >= q_len) return;  // an item past the request's tokens (a batch of fixed shape)
-  const int ntok = min(min(item[2], SHORT_CONV_TOKENS), q_len - tok0);
+  int ntok = min(min(item[2], SHORT_CONV_TOKENS), q_len - tok0);
+  if constexpr (TAPS > 0) {
+    // the item's tokens in runs of SHORT_CONV_RUN, a workgroup each
+    const int first = blockIdx.z * SHORT_CONV_RUN;
+    if (first >= ntok) return;
+    tok0 += first;
+    ntok = min(ntok - first, SHORT_CONV_RUN);
+  }
   const int c = (blockIdx.y * 256 + threadIdx.x) * V;
   if (c >= p.channels) return;
   const int slot = p.state_slots[req];
@@ -71,11 +80,12 @@ __global__ __launch_bounds__(256) void short_conv_kernel(ShortConv p) {
 #pragma unroll
     for (int k = 0; k < TAPS - 1; ++k) input(tok0 - (TAPS - 1) + k, win[k + 1]);
     // all of the item's rows are asked for before the first is used
-    float x[SHORT_CONV_TOKENS][V];
+    float x[SHORT_CONV_RUN][V];
 #pragma unroll
-    for (int i = 0; i < SHORT_CONV_TOKENS; ++i) CwVec<T, V>::load(in + (int64_t)(tok0 + min(i, ntok - 1)) * p.in_stride, x[i]);
+    for (int i = 0; i < SHORT_CONV_RUN; ++i) CwVec<T, V>::load(in + (int64_t)(tok0 + min(i, ntok - 1)) * p.in_stride, x[i]);
 #pragma unroll
-    for (int i = 0; i < SHORT_CONV_TOKENS; ++i) {
+    for (int i = 0; i < SHORT_CONV_RUN; ++i) {
+      if (i >= ntok) break;
 #pragma unroll
       for (int k = 0; k < TAPS - 1; ++k)
 #pragma unroll
@@ -89,7 +99,7 @@ __global__ __launch_bounds__(256) void short_conv_kernel(ShortConv p) {
         for (int k = 0; k < TAPS; ++k) s += w[k][v] * win[k][v];
         o[v] = p.silu ? cw_silu(s) : s;
       }
-      if (i < ntok) CwVec<T, V>::store(out + (int64_t)(tok0 + i) * p.out_stride, o);
+      CwVec<T, V>::store(out + (int64_t)(tok0 + i) * p.out_stride, o);
     }
   } else {
     for (int i = 0; i < ntok; ++i) {
@@ -123,7 +133,7 @@ static inline int short_conv_launch(const ShortConv& p, int dtype, int n_items, 
   const bool v4 = p.channels % 4 == 0 && p.in_stride % 4 == 0 && p.in_off % 4 == 0 && p.out_stride % 4 == 0 && p.out_off % 4 == 0 &&
                   !((uintptr_t)p.in & align) && !((uintptr_t)p.out & align) && p.taps >= 2 && p.taps <= 4;
   const int per = v4 ? 4 : 1;
-  dim3 grid(n_items, (p.channels + 256 * per - 1) / (256 * per)), block(256);
+  dim3 grid(n_items, (p.channels + 256 * per - 1) / (256 * per), v4 ? SHORT_CONV_TOKENS / SHORT_CONV_RUN : 1), block(256);
 #define CW_CONV(T_, V_, K_) hipLaunchKernelGGL((short_conv_kernel<T_, V_, K_>), grid, block, 0, stream, p)
 #define CW_BY_TAPS(T_)                      \
   do {                                      \

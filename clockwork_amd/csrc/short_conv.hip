@@ -63,6 +63,7 @@ struct QkvConv {
 };
 
 #define QKV_MAX_RUN SHORT_CONV_TOKENS
+#define QKV_RUN 4   // tokens of an item in the unrolled form (at most 4 taps)
 
 template <typename T, int V, int TAPS>
 __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
@@ -77,13 +78,6 @@ __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
   const int QK = p.nq + p.nk, C = QK + p.nv, half = p.rdims / 2;
   const int taps = TAPS ? TAPS : p.taps;
   float* cosines = qkv_lds + p.run * QK;
-  for (int i = tid; i < ntok * half; i += threads) {
-    const int t = i / half, e = i - t * half;
-    float s, c;
-    sincosf((float)p.positions[row0 + tok0 + t] * p.freq[e], &s, &c);
-    cosines[(2 * t) * half + e] = c * p.rot_mult;
-    cosines[(2 * t + 1) * half + e] = s * p.rot_mult;
-  }
   float* ring = nullptr;
   if (taps > 0) {
     const int slot = p.state_slots[req];
@@ -122,15 +116,20 @@ __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
         for (int k = 0; k < TAPS; ++k) w[k][v] = p.w[(int64_t)(c + v) * TAPS + k];
 #pragma unroll
       for (int k = 0; k < TAPS - 1; ++k) input(tok0 - (TAPS - 1) + k, win[k + 1]);
-      for (int t = 0; t < ntok; ++t) {
+      float x[QKV_RUN][V];   // the item's rows are asked for before the first is used
+#pragma unroll
+      for (int t = 0; t < QKV_RUN; ++t) CwVec<T, V>::load(in + (int64_t)(tok0 + min(t, ntok - 1)) * p.stride, x[t]);
+#pragma unroll
+      for (int t = 0; t < QKV_RUN; ++t) {
+        if (t >= ntok) break;
 #pragma unroll
         for (int k = 0; k < TAPS - 1; ++k)
 #pragma unroll
           for (int v = 0; v < V; ++v) win[k][v] = win[k + 1][v];
-        CwVec<T, V>::load(in + (int64_t)(tok0 + t) * p.stride, win[TAPS - 1]);
         float o[V];
 #pragma unroll
         for (int v = 0; v < V; ++v) {
+          win[TAPS - 1][v] = x[t][v];
           o[v] = 0.0f;
 #pragma unroll
           for (int k = 0; k < TAPS; ++k) o[v] += w[k][v] * win[k][v];
@@ -161,6 +160,13 @@ __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
         CwVec<float, V>::store(ring + (int64_t)((pos0 + i) % taps) * C + c, u);
       }
     }
+  }
+  for (int i = tid; i < ntok * half; i += threads) {
+    const int t = i / half, e = i - t * half;
+    float s, c;
+    sincosf((float)p.positions[row0 + tok0 + t] * p.freq[e], &s, &c);
+    cosines[(2 * t) * half + e] = c * p.rot_mult;
+    cosines[(2 * t + 1) * half + e] = s * p.rot_mult;
   }
   __syncthreads();
   const int wave = tid >> 6, lane = tid & 63, waves = threads >> 6;
@@ -212,7 +218,7 @@ static size_t qkv_lds_bytes(int run, int qk, int rdims) { return (size_t)run * (
 // Tokens a work item may hold (0: beyond the kernel). Few, so that a portion fills the chip; at least taps - 1.
 CW_EXPORT int cw_qkv_conv_run(int nq, int nk, int rdims, int taps) {
   if (nq < 1 || nk < 1 || rdims < 0 || taps < 0 || taps > SHORT_CONV_MAX_TAPS) return 0;
-  int run = taps - 1 > 4 ? taps - 1 : 4;
+  int run = taps - 1 > QKV_RUN ? taps - 1 : QKV_RUN;
   return qkv_lds_bytes(run, nq + nk, rdims) <= QKV_LDS_MOST ? run : 0;
 }
 

@@ -141,7 +141,7 @@ def _declare(name: str, lib: ctypes.CDLL) -> None:
             "cw_stream_beside_input": [P, P, P, P, P, I, I, I, I, I, P],
             "cw_relu_squared": [P, I, L, P],
             "cw_scale": [P, L, F, P],
-            "cw_join_dyt": [P, P, P, I, P, P, P, P, I, I, P, P, P, P, P, P, I, P, I, P, I, I, I, P],
+            "cw_join_dyt": [P, P, P, I, P, P, I, P, P, P, P, P, P, I, P, I, P, I, I, I, P],
             "cw_post_norm": [P, P, P, I, P, P, P, P, I, I, F, P, I, F, F, P, I, I, I, P],
             "cw_embedding_pair": [P, I, P, F, P, I, L, L, P, I, P, P, I, P, I, I, I, P],
         },
@@ -233,14 +233,14 @@ def _declare(name: str, lib: ctypes.CDLL) -> None:
             "cw_attention_workspace_floats": [I, I, I, I, I],
             "cw_attention": [I, I, P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, P, L, P],
             "cw_attention_prefill_supported": [],
-            "cw_attention_prefill_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, P, I, I, P, L, F, P],
+            "cw_attention_prefill_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, P, I, I, P, L, F, P, L, I, P],
             "cw_attention_prefill_workspace_floats": [I, I, I, I],
             "cw_attention_prefill_row_blocks_ok": [I],
             "cw_attention_decode_supported": [],
             "cw_attention_decode_gh": [I],
             "cw_attention_decode_max_splits": [],
             "cw_attention_decode_workspace_floats": [I, I, I, I],
-            "cw_attention_decode_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, F, P, L, P, I, I, I, F, P],
+            "cw_attention_decode_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, F, P, L, P, I, I, I, F, P, L, I, P],
         },
     }[name]
     for fn, argtypes in sigs.items():
@@ -1103,15 +1103,28 @@ def _zero_row(device) -> int:
     return t.data_ptr()
 
 
+def _head_gate(head_gate, n_tokens: int, heads: int) -> tuple:
+    """(address, row, first column) of an attention kernel's gates (z, offset), checked; none: zeros."""
+    if head_gate is None:
+        return None, 0, 0
+    gate, off = head_gate
+    _gpu(gate)
+    _need(gate.dim() == 2 and gate.dtype == torch.bfloat16 and gate.shape[0] >= n_tokens and 0 <= off and off + heads <= gate.shape[1],
+          "the gates must be bfloat16 [T, width] with a column a head")
+    return gate.data_ptr(), gate.shape[1], int(off)
+
+
 def prefill_attention_supported(hd: int, dtype: torch.dtype) -> bool:
     return dtype == torch.bfloat16 and bool(_load("attention", hd).cw_attention_prefill_supported())
 
 
 def attention_prefill(q, q_stride: int, out, k_cache, v_cache, block_tables, ctx_lens, cu_q, items, n_items: int,
                       nh: int, nkv: int, hd: int, block_size: int, window: int, scale: float,
-                      n_tokens: int, n_requests: int, row_blocks: int = 4, workspace=None, softcap: float = 0.0) -> None:
+                      n_tokens: int, n_requests: int, row_blocks: int = 4, workspace=None, softcap: float = 0.0,
+                      head_gate=None) -> None:
     """Portions of prompts through the bfloat16 matrix-core kernel (``softcap`` c > 0: scores are
-    squashed, c * tanh(scale * q . k / c), before the softmax); an item holds at most
+    squashed, c * tanh(scale * q . k / c), before the softmax; ``head_gate`` (z, offset): head h of token t is
+    multiplied by logistic(z[t, offset + h])); an item holds at most
     ``prefill_tokens_per_item(nh // nkv, row_blocks)`` tokens. ``row_blocks`` 2 instead of 4: smaller
     workgroups for launches with few items (head sizes up to 128). Other arguments as for ``attention``.
     An item's fourth field is ``part | parts << 8``: with parts > 1 the item stands that many times
@@ -1147,7 +1160,7 @@ def attention_prefill(q, q_stride: int, out, k_cache, v_cache, block_tables, ctx
             q.data_ptr(), int(q_stride), _ptr(out), out_stride, _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
             block_tables.shape[1], _ptr(ctx_lens), _ptr(cu_q), _ptr(items), n_items, nh, nkv, block_size,
             window, float(scale), _zero_row(out.device), int(row_blocks), int(workspace is not None), _ptr(workspace),
-            ws_floats, float(softcap), _stream()),
+            ws_floats, float(softcap), *_head_gate(head_gate, n_tokens, nh), _stream()),
         "attention_prefill_bf16",
     )
 
@@ -1181,9 +1194,9 @@ def decode_attention_workspace_floats(hd: int, n_items: int, nh: int, nkv: int, 
 def attention_decode(q, q_stride: int, out, k_cache, v_cache, block_tables, ctx_lens, cu_q, items, n_items: int,
                      nh: int, nkv: int, hd: int, block_size: int, n_splits: int, window: int, scale: float,
                      n_tokens: int, n_requests: int, workspace=None, identity: bool = False,
-                     split_keys: int = 0, max_ctx: int = 0, softcap: float = 0.0) -> None:
+                     split_keys: int = 0, max_ctx: int = 0, softcap: float = 0.0, head_gate=None) -> None:
     """Single-token items through the bfloat16 decode kernel; arguments as for ``attention``
-    (``softcap`` as for ``attention_prefill``).
+    (``softcap`` and ``head_gate`` as for ``attention_prefill``).
     With more than one split it needs a float32 ``workspace``. ``identity``: item i is request i
     with its token in row i (no other items). ``split_keys`` > 0: every split takes that many
     keys at a fixed place; no context may then be longer than ``max_ctx`` <= n_splits * split_keys."""
@@ -1221,7 +1234,7 @@ def attention_decode(q, q_stride: int, out, k_cache, v_cache, block_tables, ctx_
             q.data_ptr(), int(q_stride), _ptr(out), out_stride, _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
             block_tables.shape[1], _ptr(ctx_lens), _ptr(cu_q), _ptr(items), n_items, nh, nkv, block_size, n_splits,
             window, float(scale), _ptr(workspace), ws_floats, _zero_row(out.device), int(bool(identity)),
-            int(split_keys), int(max_ctx), float(softcap), _stream()),
+            int(split_keys), int(max_ctx), float(softcap), *_head_gate(head_gate, n_tokens, nh), _stream()),
         "attention_decode_bf16",
     )
 
@@ -2669,8 +2682,8 @@ def join_dynamic_tanh(resid, branch, b_weight, b_bias, b_alpha, weight=None, bia
     weight + bias, float32 inside. ``branch``: [T, H] in the activation type, :class:`PartialSums` or
     :class:`RoutedSum` without identity experts (both added up inside). With ``rows`` only those rows are
     made, into out[i], and resid is left alone."""
-    parts = pairs = choice = score = always = plain = None
-    n_parts = top = experts = 0
+    parts = pairs = always = plain = None
+    n_parts = top = 0
     T, H = resid.shape
     _need(resid.dtype == torch.float32, "the residual stream is float32")
     dtype = out.dtype if out is not None else None
@@ -2680,16 +2693,15 @@ def join_dynamic_tanh(resid, branch, b_weight, b_bias, b_alpha, weight=None, bia
         dtype = dtype or (torch.bfloat16 if b_weight.dtype == torch.bfloat16 else torch.float32)
         _need(tuple(parts.shape) == (n_parts, T, H) and parts.dtype == torch.float32, "partial sums must be float32 [parts, T, H]")
     elif isinstance(branch, RoutedSum):
-        pairs, choice, score, always, top, experts = branch.y, branch.choice, branch.score, branch.always, branch.top, branch.experts
+        pairs, always, top = branch.y, branch.always, branch.top
         dtype = dtype or pairs.dtype
-        _need(pairs.dtype == dtype and tuple(pairs.shape) == (T * top, H) and choice.dtype == torch.int32 and choice.numel() == T * top
-              and score.dtype == torch.float32 and score.numel() == T * top, "a routed sum has a row, a choice and a score a pair")
+        _need(pairs.dtype == dtype and tuple(pairs.shape) == (T * top, H), "a routed sum has a row a pair")
         _need(always is None or (tuple(always.shape) == (T, H) and always.dtype == dtype), "the expert of every token must be [T, H]")
     else:
         plain = branch
         dtype = dtype or plain.dtype
         _need(tuple(plain.shape) == (T, H) and plain.dtype == dtype, "the branch must be [T, H] in the activation type")
-    _gpu(resid, plain, parts, pairs, choice, score, always, b_weight, b_bias, b_alpha, weight, bias, alpha, out, rows)
+    _gpu(resid, plain, parts, pairs, always, b_weight, b_bias, b_alpha, weight, bias, alpha, out, rows)
     n = T if rows is None else rows.numel()
     if rows is not None:
         _i32(rows, n, "rows")
@@ -2699,8 +2711,8 @@ def join_dynamic_tanh(resid, branch, b_weight, b_bias, b_alpha, weight=None, bia
         _need(wt is None or (wt.numel() == H and wt.dtype == b_weight.dtype), "norm weights and biases must have the row's size and one type")
     for a in (b_alpha, alpha):
         _need(a is None or (a.dtype == torch.float32 and a.numel() == 1), "alpha must be one float32 element")
-    _check(_load("rowwise").cw_join_dyt(_ptr(resid), _ptr(plain), _ptr(parts), n_parts, _ptr(pairs), _ptr(choice), _ptr(score), _ptr(always),
-                                        int(top), int(experts), _ptr(b_weight), _ptr(b_bias), _ptr(b_alpha), _ptr(weight), _ptr(bias),
+    _check(_load("rowwise").cw_join_dyt(_ptr(resid), _ptr(plain), _ptr(parts), n_parts, _ptr(pairs), _ptr(always),
+                                        int(top), _ptr(b_weight), _ptr(b_bias), _ptr(b_alpha), _ptr(weight), _ptr(bias),
                                         _ptr(alpha), dtype_code(b_weight.dtype), _ptr(out), dtype_code(dtype), _ptr(rows), n, T, H,
                                         _stream()), "join_dynamic_tanh")
     return out

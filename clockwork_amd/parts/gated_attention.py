@@ -191,7 +191,7 @@ class GatedAttention(Part):
                                     pairing=self.pairing, norm=self.norm_order, query_temperature=s.query_temperature)
         cache = pages
         if self.plain:
-            self._attend_plain(q, out, ctx, cache, k_plane, v_plane)
+            self._attend_plain(q, out, ctx, cache, k_plane, v_plane, (proj, off + self.g_off) if self._gate_inside else None)
         else:
             items, n_items, runs = self._plan(ctx)
             ops.rows_attention(q, (q.shape[1], s.key_dim), out, (out.stride(0), s.value_dim), k_plane, v_plane,
@@ -200,13 +200,13 @@ class GatedAttention(Part):
                                mask="window" if s.window is not None else "causal", mask_size=s.window or 0,
                                keep_first=s.keep_first, softcap=s.softcap or 0.0, mfma=self.rows_mfma, key_runs=runs,
                                head_gate=(proj, off + self.g_off) if self._gate_inside else None)
-        if s.output_gate and not (self._gate_inside and not self.plain):
+        if s.output_gate and not self._gate_inside:
             bias_free = self.in_bias is None
             if not bias_free:
                 raise NotImplementedError("an output gate with a bias")
             ops.sigmoid_mul_(out, proj, off + self.g_off, group=s.value_dim if s.gate_per_head else 1)
 
-    def _attend_plain(self, q, out, ctx, cache, k_plane, v_plane) -> None:
+    def _attend_plain(self, q, out, ctx, cache, k_plane, v_plane, head_gate) -> None:
         """The kernels of plain grouped attention on the two planes (each [rows, kv_heads, size])."""
         s = self.spec
         nh, nkv, hd = s.num_heads, s.num_kv_heads, s.key_dim
@@ -216,7 +216,7 @@ class GatedAttention(Part):
             q=q, q_stride=q.shape[1], out=out, k_cache=k_plane, v_cache=v_plane,
             block_tables=ctx.block_tables[cache.group], ctx_lens=ctx.ctx_lens, cu_q=ctx.cu_q,
             nh=nh, nkv=nkv, hd=hd, block_size=cache.block_size, window=s.window or 0,
-            scale=s.scale, n_tokens=T, n_requests=ctx.num_requests, softcap=s.softcap or 0.0,
+            scale=s.scale, n_tokens=T, n_requests=ctx.num_requests, softcap=s.softcap or 0.0, head_gate=head_gate,
         )
         if plan.n_wide:
             workspace = None

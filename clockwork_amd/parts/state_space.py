@@ -121,7 +121,7 @@ class StateSpace(Part):
 
 # tokens of a segment of a selective scan, by the step's tokens: short steps are cut finer, so that they
 # have as many segments side by side
-SCAN_SEGMENTS = ((1024, 64), (256, 32), (0, 16))
+SCAN_SEGMENTS = ((1024, 32), (0, 16))
 
 
 class SelectiveScan(Part):

@@ -549,3 +549,99 @@ def random_dogudra_config(seed: int) -> dict:
             "norm": {"eps": rng.choice([1e-6, 1e-5])}, "postln_alpha": rng.choice([1.0, 1.5, 3.0]),
             "embedding": {"scale": rng.choice([1.0, 4.0]), "bigram": {"buckets": buckets, "mul_prev": rng.choice([1, 31, 997]), "mul_cur": rng.choice([1, 7, 1009])}},
             "layers": layers}
+
+
+# ------------------------------------------------------------------------------- Tufevik
+def _tufevik_memory(heads, dim, vdim, cap):
+    return {"heads": heads, "dim": dim, "vdim": vdim, "gate_cap": cap}
+
+
+def _tufevik_pair(left, right, scales, yarn=(4.0, 64, 8.0, 1.0)):
+    """``left``: heads, kv_heads, dim, vdim, taps, scale, base, rotated dims; ``right``: inner, state, taps, rank."""
+    heads, kv_heads, dim, vdim, conv, scale, base, dims = left
+    rot = {"base": base, "dims": dims}
+    if yarn is not None:
+        rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), yarn))
+    return {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv, "scale": scale, "rot": rot},
+            "right": dict(zip(("inner", "state", "conv", "dt_rank"), right)), "left_scale": scales[0], "right_scale": scales[1]}
+
+
+def _tufevik_moe(ff, experts, top):
+    return {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+
+
+def _tufevik_dense(ff):
+    return {"kind": "dense", "ff": ff}
+
+
+# both mixers, values of another size than keys, dense, routed and no feed-forward
+TUFEVIK_A = {
+    "architecture": "Tufevik", "vocab": 211, "width": 96, "norm": {"eps": 1e-5}, "embedding": {"scale": 3.0},
+    "layers": [
+        {"type": "parallel", "mixer": _tufevik_pair((6, 2, 24, 40, 3, 0.3, 500.0, 16), (80, 12, 4, 10), (0.6, 1.3)), "mlp": _tufevik_moe(40, 6, 3)},
+        {"type": "mlstm", "mixer": _tufevik_memory(3, 24, 40, 9.0), "mlp": _tufevik_dense(120)},
+        {"type": "parallel", "mixer": _tufevik_pair((4, 4, 32, 32, 2, 0.2, 10000.0, 32), (64, 8, 2, 8), (1.0, 0.5), (8.0, 256, 16.0, 2.0)), "mlp": None},
+        {"type": "mlstm", "mixer": _tufevik_memory(2, 64, 16, 20.0), "mlp": _tufevik_moe(24, 4, 1)},
+    ],
+}
+# a width that is no multiple of 8, sizes of 1 and odd ones, one tap and many, no rotation, unscaled rotation,
+# columns that begin at no multiple of 16 bytes, every expert chosen
+TUFEVIK_B = {
+    "architecture": "Tufevik", "vocab": 90, "width": 100, "norm": {"eps": 1e-4}, "embedding": {"scale": 1.0},
+    "layers": [
+        {"type": "parallel", "mixer": _tufevik_pair((3, 1, 10, 7, 1, 0.5, 100.0, 0), (33, 5, 6, 3), (1.0, 1.0), None), "mlp": _tufevik_moe(30, 3, 3)},
+        {"type": "mlstm", "mixer": _tufevik_memory(1, 1, 1, 4.0), "mlp": _tufevik_dense(70)},
+        {"type": "parallel", "mixer": _tufevik_pair((1, 1, 6, 2, 9, 1.0, 10.0, 6), (10, 1, 1, 1), (2.0, 0.3), None), "mlp": _tufevik_dense(36)},
+        {"type": "mlstm", "mixer": _tufevik_memory(5, 7, 9, 15.0), "mlp": None},
+    ],
+}
+# matrix memories alone (no pages at all), of two sizes
+TUFEVIK_C = {
+    "architecture": "Tufevik", "vocab": 130, "width": 64, "norm": {"eps": 1e-6}, "embedding": {"scale": 8.0},
+    "layers": [
+        {"type": "mlstm", "mixer": _tufevik_memory(4, 16, 32, 12.0), "mlp": _tufevik_dense(96)},
+        {"type": "mlstm", "mixer": _tufevik_memory(2, 48, 80, 15.0), "mlp": _tufevik_moe(64, 8, 2)},
+    ],
+}
+# parallel layers alone, head sizes of the kernels for plain grouped attention and for paged rows
+TUFEVIK_D = {
+    "architecture": "Tufevik", "vocab": 150, "width": 128, "norm": {"eps": 1e-6}, "embedding": {"scale": 5.0},
+    "layers": [
+        {"type": "parallel", "mixer": _tufevik_pair((8, 2, 64, 64, 4, 0.1, 10000.0, 64), (256, 16, 4, 16), (0.7, 0.7)), "mlp": _tufevik_moe(64, 8, 4)},
+        {"type": "parallel", "mixer": _tufevik_pair((4, 1, 64, 128, 4, 0.15, 10000.0, 32), (128, 40, 3, 24), (0.9, 0.4), (2.0, 128, 4.0, 0.5)), "mlp": _tufevik_dense(64)},
+    ],
+}
+TUFEVIK_CONFIGS = {"TA": (TUFEVIK_A, 71, 8), "TB": (TUFEVIK_B, 72, 16), "TC": (TUFEVIK_C, 73, 4), "TD": (TUFEVIK_D, 74, 8)}
+
+
+def random_tufevik_config(seed: int) -> dict:
+    """A model of the design drawn at random: two to six layers that share nothing, head, state and inner
+    sizes that the matrix-core kernels take and ones they do not, one to five taps."""
+    import random
+
+    rng = random.Random(seed)
+    layers = []
+    for _ in range(rng.randint(2, 6)):
+        kind = rng.random()
+        if kind < 0.15:
+            mlp = None
+        elif kind < 0.45:
+            mlp = _tufevik_dense(rng.choice([64, 100, 192, 256]))
+        else:
+            experts = rng.choice([1, 2, 5, 8, 16])
+            mlp = _tufevik_moe(rng.choice([40, 64, 88, 128]), experts, rng.randint(1, min(4, experts)))
+        if rng.random() < 0.5:
+            mixer = _tufevik_memory(rng.choice([1, 2, 3, 4, 8]), rng.choice([8, 16, 20, 24, 64, 128]), rng.choice([8, 20, 32, 64, 96, 136]),
+                                    rng.choice([5.0, 15.0, 30.0]))
+            layers.append({"type": "mlstm", "mixer": mixer, "mlp": mlp})
+            continue
+        kv_heads = rng.choice([1, 2, 3, 4])
+        dim = rng.choice([16, 24, 32, 64, 128])
+        vdim = dim if rng.random() < 0.5 else rng.choice([16, 24, 40, 64, 128])
+        left = (kv_heads * rng.choice([1, 2, 4]), kv_heads, dim, vdim, rng.choice([1, 2, 3, 4, 5]), dim ** -0.5 * rng.choice([0.5, 1.0, 2.0]),
+                rng.choice([100.0, 10000.0, 5e5]), rng.choice([0, dim // 2, dim]))
+        right = (rng.choice([48, 100, 192, 256]), rng.choice([4, 8, 12, 16, 24, 40, 64]), rng.choice([1, 2, 3, 4, 5]), rng.choice([3, 8, 16, 40]))
+        yarn = rng.choice([None, (4.0, 64, 8.0, 1.0), (16.0, 512, 32.0, 1.0), (1.0, 32, 2.0, 1.0)])
+        layers.append({"type": "parallel", "mixer": _tufevik_pair(left, right, (rng.choice([0.3, 1.0, 1.5]), rng.choice([0.4, 1.0, 2.0])), yarn), "mlp": mlp})
+    return {"architecture": "Tufevik", "vocab": rng.choice([300, 500, 1000]), "width": rng.choice([128, 192, 264, 384]),
+            "norm": {"eps": rng.choice([1e-6, 1e-5])}, "embedding": {"scale": rng.choice([1.0, 6.0])}, "layers": layers}
