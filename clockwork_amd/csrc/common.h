@@ -74,8 +74,31 @@ __device__ __forceinline__ float cw_gelu_tanh(float z) {
   return z / (1.0f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
 }
 
-__device__ __forceinline__ float cw_silu(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float cw_logistic(float z) { return 1.0f / (1.0f + expf(-z)); }
+// Functions from the bare exp2, log2 and reciprocal instructions: a few units in the last place, and a
+// fraction of the code of the library's (a kernel that runs for microseconds waits for its own code).
+__device__ __forceinline__ float cw_exp_quick(float z) { return __builtin_amdgcn_exp2f(1.44269504f * z); }
+__device__ __forceinline__ float cw_logistic(float z) { return __builtin_amdgcn_rcpf(1.0f + cw_exp_quick(-z)); }
+__device__ __forceinline__ float cw_silu(float z) { return z * cw_logistic(z); }
+// tanh: a power series for small z, else (1 - e) / (1 + e) with e = exp(-2 |z|)
+__device__ __forceinline__ float cw_tanh_quick(float z) {
+  const float s = z * z, e = cw_exp_quick(-2.0f * fabsf(z));
+  const float series = z * (1.0f + s * (-0.333333333f + s * (0.133333333f + s * (-0.053968254f + s * 0.021869489f))));
+  const float direct = copysignf((1.0f - e) * __builtin_amdgcn_rcpf(1.0f + e), z);
+  return s < 0.0625f ? series : direct;
+}
+// Sine and cosine of an angle in radians, |a| up to 2^20: quarter turns from a product with 2 / pi in two
+// parts, then the Taylor series on [-pi/4, pi/4].
+__device__ __forceinline__ void cw_sincos_quick(float a, float& s, float& c) {
+  const float hi = a * 0.636619772f, lo = fmaf(a, 0.636619772f, -hi) + a * 2.56825533e-8f;
+  const float n = rintf(hi);
+  const float r = ((hi - n) + lo) * 1.57079633f, q = r * r;
+  const float sn = r * (1.0f + q * (-0.166666667f + q * (8.33333333e-3f + q * (-1.98412698e-4f + q * 2.75573192e-6f))));
+  const float cs = 1.0f + q * (-0.5f + q * (4.16666667e-2f + q * (-1.38888889e-3f + q * 2.48015873e-5f)));
+  const int k = (int)n & 3;
+  const float u = k & 1 ? cs : sn, v = k & 1 ? sn : cs;
+  s = k & 2 ? -u : u;
+  c = (k + 1) & 2 ? -v : v;
+}
 __device__ __forceinline__ float cw_softplus(float z) { return z > 0.0f ? z + log1pf(expf(-z)) : log1pf(expf(z)); }
 // The same from the bare exp2 and log2 instructions: max(z, 0) + ln(1 + e), e = exp(-|z|). ln(1 + e) is a
 // short power series for small e, where 1 + e would lose its digits, and else ln(u) e / (u - 1) with u = 1 + e

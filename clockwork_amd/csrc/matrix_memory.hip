@@ -42,7 +42,7 @@ struct MmParams {
   const void* gate_w;      // [2 * heads, width]: the rows of i, then those of f
   const float* gate_b;     // [2 * heads]
   int width;
-  float cap, q_scale;
+  float cap, inv_cap, q_scale;
   float* gates;            // [T, 2 * heads] i and f (not for single tokens)
   float* state;
   int64_t state_stride;
@@ -61,8 +61,11 @@ struct MmParams {
   int heads, D, V, n_tokens;
 };
 
-__device__ __forceinline__ float mm_log_input(float z, float cap) { return cap * tanhf(z / cap); }
-__device__ __forceinline__ float mm_log_forget(float z, float cap) { return -cw_softplus_quick(-(cap * tanhf(z / cap))); }
+// the capped logarithm of a gate: of the input gate as it is, of the forget gate through log logistic
+__device__ __forceinline__ float mm_log_gate(float z, float cap, float inv_cap, bool forget) {
+  const float u = cap * cw_tanh_quick(z * inv_cap);
+  return forget ? -cw_softplus_quick(-u) : u;
+}
 __host__ __device__ inline int mm_round(int n, int to) { return (n + to - 1) / to * to; }
 // n and m of a head as the token at position ``pos`` leaves them
 __device__ __forceinline__ float* mm_norm_at(const MmParams& p, float* slot, int pos, int h) {
@@ -88,7 +91,7 @@ __global__ __launch_bounds__(MM_GATE_WAVES * 64) void mm_gate_kernel(MmParams p,
   }
   const int tiles = min(4, (G - g0 + 15) / 16);
   if constexpr (sizeof(T) == 2) {
-#pragma unroll 4
+#pragma unroll 3
     for (int k = wave * 32; k < p.width; k += MM_GATE_WAVES * 32) {
       const int kk = k + kq * 8;
       union { u32x4_t u; bf16x8_t v; uint16_t s[8]; } a, b[4];
@@ -136,7 +139,7 @@ __global__ __launch_bounds__(MM_GATE_WAVES * 64) void mm_gate_kernel(MmParams p,
     const int g = g0 + j * 16 + kq * 4 + e;
     if (g < G) {
       const float z = sum[e] + p.gate_b[g];
-      p.gates[(int64_t)(t0 + i) * G + g] = g < p.heads ? mm_log_input(z, p.cap) : mm_log_forget(z, p.cap);
+      p.gates[(int64_t)(t0 + i) * G + g] = mm_log_gate(z, p.cap, p.inv_cap, g >= p.heads);
     }
   }
 }
@@ -144,47 +147,73 @@ __global__ __launch_bounds__(MM_GATE_WAVES * 64) void mm_gate_kernel(MmParams p,
 // ---------------------------------------------------------------- chunks
 template <typename T> struct MmPad { static constexpr int V = sizeof(T) == 2 ? 8 : 4; };
 
-// Rows of an operand in LDS: ``width`` elements, zeros past the operand's ``n`` and past the ``nt`` tokens.
-// Loads are never conditional (a clamped address, zeros chosen afterwards), so several are on their way at once.
-template <typename T, int THREADS>
-__device__ __forceinline__ void mm_stage(T* dst, int dst_stride, int width, const T* src, int64_t src_stride, int n, int nt, int rows, bool vec) {
-  constexpr int V = MmPad<T>::V;
-  if (vec) {
-    const int per = width / V, total = rows * per;
-#pragma unroll 1
-    for (int i0 = threadIdx.x; i0 < total; i0 += 4 * THREADS) {
-      u32x4_t v[4];
-      int at[4];
+// An operand's rows on their way to LDS: ``width`` elements, zeros past the operand's ``n`` and past the ``nt``
+// tokens. LANES neighbouring threads share a row, U rows a thread make a batch. The first batches of all
+// operands are asked for (``load``) before any of them is waited for (``store``, which also fetches what is
+// left). Loads are never conditional: a clamped address, zeros chosen afterwards.
+// ``ACROSS``: LDS holds the operand's columns side by side, each with its tokens (element e of row t at
+// dst[e * dst_stride + t]), so that a lane reads four neighbouring tokens of a column at once.
+template <typename T, int THREADS, int LANES, int U, bool ACROSS>
+struct MmRows {
+  static constexpr int V = MmPad<T>::V, ROWS = THREADS / LANES;
+  u32x4_t v[U];
+  __device__ __forceinline__ void load(const T* src, int64_t src_stride, int e, int t0, int n, int nt) {
+    const T* at = src + min(e, n - V);
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
-        const int i = min(i0 + u * THREADS, total - 1), t = i / per, e = (i - t * per) * V;
-        at[u] = t * dst_stride + e;
-        const u32x4_t got = *reinterpret_cast<const u32x4_t*>(src + (int64_t)min(t, nt - 1) * src_stride + min(e, n - V));
-        v[u] = (t < nt && e < n) ? got : (u32x4_t){0u, 0u, 0u, 0u};
+    for (int u = 0; u < U; ++u) v[u] = *reinterpret_cast<const u32x4_t*>(at + (int64_t)min(t0 + u * ROWS, nt - 1) * src_stride);
+  }
+  __device__ __forceinline__ void first(const T* src, int64_t src_stride, int n, int nt, bool vec) {
+    if (vec) load(src, src_stride, (threadIdx.x % LANES) * V, threadIdx.x / LANES, n, nt);
+  }
+  __device__ __forceinline__ void put(T* dst, int dst_stride, int e, int t0, int n, int nt, int rows, int width) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int t = t0 + u * ROWS;
+      if (t < rows && e < width) {
+        const u32x4_t z = (t < nt && e < n) ? v[u] : (u32x4_t){0u, 0u, 0u, 0u};
+        if constexpr (!ACROSS) {
+          *reinterpret_cast<u32x4_t*>(dst + t * dst_stride + e) = z;
+        } else {
+          union { u32x4_t w; T x[V]; } parts;
+          parts.w = z;
+#pragma unroll
+          for (int i = 0; i < V; ++i) dst[(e + i) * dst_stride + t] = parts.x[i];
+        }
       }
-#pragma unroll
-      for (int u = 0; u < 4; ++u) *reinterpret_cast<u32x4_t*>(dst + at[u]) = v[u];
-    }
-  } else {
-    for (int i = threadIdx.x; i < rows * width; i += THREADS) {
-      const int t = i / width, e = i - t * width;
-      dst[t * dst_stride + e] = (t < nt && e < n) ? src[(int64_t)t * src_stride + e] : cw_from_float<T>(0.0f);
     }
   }
-}
+  __device__ __forceinline__ void store(T* dst, int dst_stride, int width, const T* src, int64_t src_stride, int n, int nt, int rows, bool vec) {
+    const int r = threadIdx.x / LANES, l = threadIdx.x % LANES;
+    if (vec) {
+      put(dst, dst_stride, l * V, r, n, nt, rows, width);
+#pragma unroll 1
+      for (int e = l * V; e < width; e += LANES * V)
+#pragma unroll 1
+        for (int t0 = r + (e == l * V ? U * ROWS : 0); t0 < rows; t0 += U * ROWS) {
+          load(src, src_stride, e, t0, n, nt);
+          put(dst, dst_stride, e, t0, n, nt, rows, width);
+        }
+    } else {
+#pragma unroll 1
+      for (int t = r; t < rows; t += ROWS)
+#pragma unroll 1
+        for (int e = l; e < width; e += LANES)
+          dst[ACROSS ? e * dst_stride + t : t * dst_stride + e] = (t < nt && e < n) ? src[(int64_t)t * src_stride + e] : cw_from_float<T>(0.0f);
+    }
+  }
+};
 
-// A lane a token of the chunk (the first wave): F, the running sum of f, and b = i - F (MM_NONE past the
-// chunk's tokens, where F stays what it was).
-__device__ __forceinline__ void mm_gates(const MmParams& p, int64_t row, bool live, int h, float& F, float& b) {
+// A lane a token of the chunk (the first wave), from its i and f: F, the running sum of f, and b = i - F
+// (MM_NONE past the chunk's tokens, where F stays what it was).
+__device__ __forceinline__ void mm_gates(float gi, float gf, bool live, float& F, float& b) {
   const int lane = threadIdx.x;
-  const float* g = p.gates + row * (2 * p.heads);
-  F = live ? g[p.heads + h] : 0.0f;
+  F = live ? gf : 0.0f;
 #pragma unroll
   for (int off = 1; off < 64; off <<= 1) {
     const float o = __shfl_up(F, off, 64);
     if (lane >= off) F += o;
   }
-  b = live ? g[h] - F : MM_NONE;
+  b = live ? gi - F : MM_NONE;
 }
 
 template <typename T, int Q>
@@ -198,47 +227,65 @@ __global__ __launch_bounds__(Q * 4) void mm_chunk_state_kernel(MmParams p, int v
   if (tok0 >= q_len) return;  // a chunk past the request's tokens (a batch of fixed shape)
   const int nt = min(min(item[2], Q), q_len - tok0);
   const int D = p.D, V = min(MM_COLS, p.V - v0), Dp = mm_round(D, 16), Vp = mm_round(V, 16);
-  const int SK = Dp + MmPad<T>::V, SV = MM_COLS + MmPad<T>::V;
-  T* Ks = (T*)smem;                // [Q][SK]
-  T* Vs = Ks + Q * SK;             // [Q][SV]
+  constexpr int ST = Q + 4;
+  T* Ks = (T*)smem;                // [Dp][ST]
+  T* Vs = Ks + Dp * ST;            // [MM_COLS][ST]
   const T* rows = (const T*)p.proj + (int64_t)(row0 + tok0) * p.stride;
+  const float* gates = p.gates + (int64_t)(row0 + tok0 + min((int)threadIdx.x, nt - 1)) * (2 * p.heads);
+  const float gi = threadIdx.x < 64 ? gates[h] : 0.0f, gf = threadIdx.x < 64 ? gates[p.heads + h] : 0.0f;
+  const T *k_rows = rows + p.k_off + h * D, *v_rows = rows + p.v_off + h * p.V + v0;
+  MmRows<T, THREADS, 16, 4, true> ks;
+  MmRows<T, THREADS, sizeof(T) == 2 ? 8 : 16, 2, true> vs;
+  ks.first(k_rows, p.stride, D, nt, vec);
+  vs.first(v_rows, p.stride, V, nt, vec);
+  ks.store(Ks, ST, Dp, k_rows, p.stride, D, nt, Q, vec);
+  vs.store(Vs, ST, Vp, v_rows, p.stride, V, nt, Q, vec);
   if (threadIdx.x < 64) {
     const int t = threadIdx.x;
     float F, b;
-    mm_gates(p, row0 + tok0 + min(t, nt - 1), t < nt, h, F, b);
+    mm_gates(gi, gf, t < nt, F, b);
     const float most = cw_wave_max(b);
-    wt[t] = t < nt ? expf(b - most) : 0.0f;
+    wt[t] = t < nt ? cw_exp_quick(b - most) : 0.0f;
     if (t == 63 && blockIdx.z == 0) {
       p.added_n[((int64_t)blockIdx.x * p.heads + h) * (D + 1) + D] = F + most;
       p.chunk_f[(int64_t)blockIdx.x * p.heads + h] = F;
     }
   }
-  mm_stage<T, THREADS>(Ks, SK, Dp, rows + p.k_off + h * D, p.stride, D, nt, Q, vec);
-  mm_stage<T, THREADS>(Vs, SV, Vp, rows + p.v_off + h * p.V + v0, p.stride, V, nt, Q, vec);
   __syncthreads();
   if (blockIdx.z == 0) {
     float* an = p.added_n + ((int64_t)blockIdx.x * p.heads + h) * (D + 1);
     for (int d = threadIdx.x; d < D; d += THREADS) {
       float s = 0.0f;
-      for (int t = 0; t < nt; ++t) s += wt[t] * cw_to_float(Ks[t * SK + d]);
+#pragma unroll 4
+      for (int t = 0; t < Q; t += 4) {   // zeros past the chunk's tokens
+        float k[4];
+        CwVec<T, 4>::load(Ks + d * ST + t, k);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) s += wt[t + u] * k[u];
+      }
       an[d] = s;
     }
   }
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, i = lane & 15, kq = lane >> 4;
   float* out = p.added + ((int64_t)blockIdx.x * p.heads + h) * D * p.V + v0;
-  const int v_tiles = Vp / 16, k_end = mm_round(nt, 4);
+  const int v_tiles = Vp / 16, k_end = mm_round(nt, 16);
+  // a lane quarter takes four neighbouring tokens, one a product: which tokens meet in a product is all one
   for (int tn = wave; tn < Dp / 16; tn += WAVES) {
     f32x4_t acc[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[j] = (f32x4_t){0.0f, 0.0f, 0.0f, 0.0f};
-#pragma unroll 4
-    for (int k = 0; k < k_end; k += 4) {
-      const int t = k + kq;
-      const float a = cw_to_float(Ks[t * SK + tn * 16 + i]) * wt[t];
+#pragma unroll 2
+    for (int k = 0; k < k_end; k += 16) {
+      const int t = k + kq * 4;
+      float a[4], b[4][4];
+      CwVec<T, 4>::load(Ks + (tn * 16 + i) * ST + t, a);
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int col = min(j, v_tiles - 1) * 16 + i;
-        acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, cw_to_float(Vs[t * SV + col]), acc[j], 0, 0, 0);
+      for (int j = 0; j < 4; ++j) CwVec<T, 4>::load(Vs + (min(j, v_tiles - 1) * 16 + i) * ST + t, b[j]);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        a[u] *= wt[t + u];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[u], b[j][u], acc[j], 0, 0, 0);
       }
     }
 #pragma unroll
@@ -277,18 +324,28 @@ __global__ __launch_bounds__(256) void mm_carry_kernel(MmParams p) {
   if (norm) {
     for (int d = threadIdx.x; d < mm_round(p.D + 1, 256); d += 256) {
       float n = d < p.D ? before[d] : 0.0f, mm = m;
-      for (int c = begin; c < end; ++c) {
-        float* an = p.added_n + ((int64_t)c * p.heads + h) * (p.D + 1);
-        const float f = p.chunk_f[(int64_t)c * p.heads + h], most = an[p.D];
-        const float next = fmaxf(mm + f, most);
-        if (d < p.D) {
-          const float add = an[d];
-          an[d] = n;
-          n = expf(mm + f - next) * n + expf(most - next) * add;
-        } else if (d == p.D) {
-          p.start_m[(int64_t)c * p.heads + h] = mm;
+      for (int c0 = begin; c0 < end; c0 += 16) {
+        float add[16], f[16], most[16];   // sixteen chunks' loads side by side
+#pragma unroll
+        for (int u = 0; u < 16; ++u) {
+          const int64_t ch = (int64_t)min(c0 + u, end - 1) * p.heads + h;
+          add[u] = p.added_n[ch * (p.D + 1) + min(d, p.D)];
+          most[u] = p.added_n[ch * (p.D + 1) + p.D];
+          f[u] = p.chunk_f[ch];
         }
-        mm = next;
+#pragma unroll
+        for (int u = 0; u < 16; ++u) {
+          if (c0 + u >= end) continue;
+          const int64_t ch = (int64_t)(c0 + u) * p.heads + h;
+          const float next = fmaxf(mm + f[u], most[u]);
+          if (d < p.D) {
+            p.added_n[ch * (p.D + 1) + d] = n;
+            n = cw_exp_quick(mm + f[u] - next) * n + cw_exp_quick(most[u] - next) * add[u];
+          } else if (d == p.D) {
+            p.start_m[ch] = mm;
+          }
+          mm = next;
+        }
       }
       float* last = p.last + ((int64_t)r * p.heads + h) * (p.D + 1);
       if (d < p.D) last[d] = n;
@@ -314,7 +371,7 @@ __global__ __launch_bounds__(256) void mm_carry_kernel(MmParams p) {
       if (c0 + u < end) {
         CwVec<float, N>::store(p.added + ((int64_t)(c0 + u) * p.heads + h) * DV + e, S);
         const float next = fmaxf(m + f[u], most[u]);
-        const float keep = expf(m + f[u] - next), take = expf(most[u] - next);
+        const float keep = cw_exp_quick(m + f[u] - next), take = cw_exp_quick(most[u] - next);
 #pragma unroll
         for (int v = 0; v < N; ++v) S[v] = keep * S[v] + take * add[u][v];
         m = next;
@@ -343,18 +400,18 @@ template <typename T, int Q>
 __global__ __launch_bounds__(Q * 4) void mm_chunk_out_kernel(MmParams p, int vec) {
   extern __shared__ __align__(16) unsigned char smem[];
   __shared__ float Fs[64], bs[64], Ms[64], den[Q], ns[MM_MAX_DIM];
-  constexpr int THREADS = Q * 4, SW = Q + 4, SS = MM_COLS + 4;
+  constexpr int THREADS = Q * 4, SW = Q + 4, ST = Q + 4;
   const int* item = p.items + 4 * (int64_t)blockIdx.x;
   const int h = blockIdx.y, req = item[0], tok0 = item[1], v0 = blockIdx.z * MM_COLS;
   const int row0 = p.cu_q[req], q_len = p.cu_q[req + 1] - row0;
   if (tok0 >= q_len) return;
   const int nt = min(min(item[2], Q), q_len - tok0);
   const int D = p.D, V = min(MM_COLS, p.V - v0), NK = mm_round(D, 32), Vp = mm_round(V, 16);
-  const int SK = NK + MmPad<T>::V, SV = MM_COLS + MmPad<T>::V;
-  T* Qs = (T*)smem;                    // [Q][SK]
-  T* Vs = Qs + Q * SK;                 // [Q][SV]
-  float* Ss = (float*)(Vs + Q * SV);   // [NK][SS]
-  T* Ks = (T*)(Ss + NK * SS);          // [Q][SK], then the weights of the tokens, float32 [Q][SW]
+  const int SK = NK + MmPad<T>::V, SS = NK + 4;
+  T* Qs = (T*)smem;                         // [Q][SK]
+  T* Vs = Qs + Q * SK;                      // [MM_COLS][ST]
+  float* Ss = (float*)(Vs + MM_COLS * ST);  // [MM_COLS][SS]
+  T* Ks = (T*)(Ss + MM_COLS * SS);          // [Q][SK], then the weights of the tokens, float32 [Q][SW]
   float* Ws = (float*)Ks;
   const T* rows = (const T*)p.proj + (int64_t)(row0 + tok0) * p.stride;
   const float* start = p.added + ((int64_t)blockIdx.x * p.heads + h) * D * p.V + v0;
@@ -368,10 +425,28 @@ __global__ __launch_bounds__(Q * 4) void mm_chunk_out_kernel(MmParams p, int vec
     const float* last = p.last + ((int64_t)req * p.heads + h) * (D + 1);
     for (int d = threadIdx.x; d <= D; d += THREADS) to[d] = last[d];
   }
+  const float* gates = p.gates + (int64_t)(row0 + tok0 + min((int)threadIdx.x, nt - 1)) * (2 * p.heads);
+  const float gi = threadIdx.x < 64 ? gates[h] : 0.0f, gf = threadIdx.x < 64 ? gates[p.heads + h] : 0.0f;
+  const T *q_rows = rows + p.q_off + h * D, *k_rows = rows + p.k_off + h * D, *v_rows = rows + p.v_off + h * p.V + v0;
+  const bool vec_s = !((p.V | V) & 3);
+  MmRows<T, THREADS, 16, 4, false> qs, ks;
+  MmRows<T, THREADS, sizeof(T) == 2 ? 8 : 16, 2, true> vs;
+  MmRows<float, THREADS, 16, 8, true> ss;
+  qs.first(q_rows, p.stride, D, nt, vec);
+  ks.first(k_rows, p.stride, D, nt, vec);
+  vs.first(v_rows, p.stride, V, nt, vec);
+  ss.first(start, p.V, V, D, vec_s);
+  const float n_mine = start_n[min((int)threadIdx.x, D - 1)];
+  if (threadIdx.x < NK) ns[threadIdx.x] = threadIdx.x < D ? n_mine : 0.0f;
+  for (int d = threadIdx.x + THREADS; d < NK; d += THREADS) ns[d] = d < D ? start_n[d] : 0.0f;
+  qs.store(Qs, SK, NK, q_rows, p.stride, D, nt, Q, vec);
+  ks.store(Ks, SK, NK, k_rows, p.stride, D, nt, Q, vec);
+  vs.store(Vs, ST, Vp, v_rows, p.stride, V, nt, Q, vec);
+  ss.store(Ss, SS, MM_COLS, start, p.V, V, D, NK, vec_s);   // (a row of the start state is p.V floats)
   if (threadIdx.x < 64) {
     const int t = threadIdx.x;
     float F, b;
-    mm_gates(p, row0 + tok0 + min(t, nt - 1), t < nt, h, F, b);
+    mm_gates(gi, gf, t < nt, F, b);
     float M = fmaxf(m_start, b);
 #pragma unroll
     for (int off = 1; off < 64; off <<= 1) {
@@ -381,33 +456,6 @@ __global__ __launch_bounds__(Q * 4) void mm_chunk_out_kernel(MmParams p, int vec
     Fs[t] = F;
     bs[t] = b;
     Ms[t] = M;
-  }
-  for (int d = threadIdx.x; d < NK; d += THREADS) ns[d] = d < D ? start_n[d] : 0.0f;
-  mm_stage<T, THREADS>(Qs, SK, NK, rows + p.q_off + h * D, p.stride, D, nt, Q, vec);
-  mm_stage<T, THREADS>(Ks, SK, NK, rows + p.k_off + h * D, p.stride, D, nt, Q, vec);
-  mm_stage<T, THREADS>(Vs, SV, Vp, rows + p.v_off + h * p.V + v0, p.stride, V, nt, Q, vec);
-  // the start state's columns (a row of it is p.V floats)
-  if (!((p.V | V) & 3)) {
-#pragma unroll 1
-    for (int i0 = threadIdx.x; i0 < NK * (MM_COLS / 4); i0 += 8 * THREADS) {
-      f32x4_t v[8];
-#pragma unroll
-      for (int u = 0; u < 8; ++u) {
-        const int i = i0 + u * THREADS, d = i / (MM_COLS / 4), c = (i - d * (MM_COLS / 4)) * 4;
-        const f32x4_t got = *reinterpret_cast<const f32x4_t*>(start + (int64_t)min(d, D - 1) * p.V + min(c, V - 4));
-        v[u] = (d < D && c < V) ? got : (f32x4_t){0.0f, 0.0f, 0.0f, 0.0f};
-      }
-#pragma unroll
-      for (int u = 0; u < 8; ++u) {
-        const int i = i0 + u * THREADS, d = i / (MM_COLS / 4), c = (i - d * (MM_COLS / 4)) * 4;
-        if (d < NK) *reinterpret_cast<f32x4_t*>(Ss + d * SS + c) = v[u];
-      }
-    }
-  } else {
-    for (int i = threadIdx.x; i < NK * MM_COLS; i += THREADS) {
-      const int d = i / MM_COLS, c = i - d * MM_COLS;
-      Ss[d * SS + c] = (d < D && c < V) ? start[(int64_t)d * p.V + c] : 0.0f;
-    }
   }
   __syncthreads();
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, i = lane & 15, kq = lane >> 4;
@@ -422,7 +470,7 @@ __global__ __launch_bounds__(Q * 4) void mm_chunk_out_kernel(MmParams p, int vec
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int t = wave * 16 + kq * 4 + e;
-        m[j][e] = t >= s ? sc[e] * p.q_scale * expf(bs[s] - Ms[t]) : 0.0f;
+        m[j][e] = t >= s ? sc[e] * p.q_scale * cw_exp_quick(bs[s] - Ms[t]) : 0.0f;
       }
     }
   }
@@ -439,10 +487,21 @@ __global__ __launch_bounds__(Q * 4) void mm_chunk_out_kernel(MmParams p, int vec
     // four lanes a token: n . q of the start and of the chunk's own tokens, and the denominator
     const int t = wave * 16 + i;
     float a = 0.0f, b = 0.0f;
-    for (int d = kq; d < D; d += 4) a += cw_to_float(qrow[d]) * ns[d];
-    for (int s = kq; s < (wave + 1) * 16; s += 4) b += wrow[s];
-    const float nq = cw_quad_sum(a * (p.q_scale * expf(m_start - Ms[t])) + b);
-    if (kq == 0) den[t] = 1.0f / (fmaxf(fabsf(nq), expf(-(Fs[t] + Ms[t]))) + MM_EPS);
+#pragma unroll 4
+    for (int d = kq * 4; d < NK; d += 16) {   // zeros past D
+      float q[4];
+      CwVec<T, 4>::load(qrow + d, q);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) a += q[u] * ns[d + u];
+    }
+#pragma unroll
+    for (int s = kq * 4; s < Q; s += 16) {    // zeros past the token's own group
+      float w[4];
+      CwVec<float, 4>::load(wrow + s, w);
+      b += (w[0] + w[1]) + (w[2] + w[3]);
+    }
+    const float nq = cw_quad_sum(a * (p.q_scale * cw_exp_quick(m_start - Ms[t])) + b);
+    if (kq == 0) den[t] = __builtin_amdgcn_rcpf(fmaxf(fabsf(nq), cw_exp_quick(-(Fs[t] + Ms[t]))) + MM_EPS);
   }
   __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront", "local");
   __builtin_amdgcn_wave_barrier();
@@ -455,23 +514,33 @@ __global__ __launch_bounds__(Q * 4) void mm_chunk_out_kernel(MmParams p, int vec
     acc[j] = (f32x4_t){0.0f, 0.0f, 0.0f, 0.0f};
     col[j] = min(j, v_tiles - 1) * 16 + i;
   }
-#pragma unroll 4
-  for (int k = 0; k < NK; k += 4) {
-    const float a = cw_to_float(qrow[k + kq]);
+#pragma unroll 2
+  for (int k = kq * 4; k < NK; k += 16) {   // (a lane quarter takes four neighbouring elements, one a product)
+    float a[4], b[4][4];
+    CwVec<T, 4>::load(qrow + k, a);
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, Ss[(k + kq) * SS + col[j]], acc[j], 0, 0, 0);
+    for (int j = 0; j < 4; ++j) CwVec<float, 4>::load(Ss + col[j] * SS + k, b[j]);
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[u], b[j][u], acc[j], 0, 0, 0);
   }
 #pragma unroll
   for (int e = 0; e < 4; ++e) {
-    const float g = p.q_scale * expf(m_start - Ms[wave * 16 + kq * 4 + e]);
+    const float g = p.q_scale * cw_exp_quick(m_start - Ms[wave * 16 + kq * 4 + e]);
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[j][e] *= g;
   }
-#pragma unroll 4
-  for (int k = 0; k < k_end; k += 4) {
-    const float a = wrow[k + kq];
+#pragma unroll 1
+  for (int k = kq * 4; k < k_end; k += 16) {
+    float a[4], b[4][4];
+    CwVec<float, 4>::load(wrow + k, a);
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, cw_to_float(Vs[(k + kq) * SV + col[j]]), acc[j], 0, 0, 0);
+    for (int j = 0; j < 4; ++j) CwVec<T, 4>::load(Vs + col[j] * ST + k, b[j]);
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[u], b[j][u], acc[j], 0, 0, 0);
   }
 #pragma unroll
   for (int e = 0; e < 4; ++e) {
@@ -553,9 +622,9 @@ __global__ __launch_bounds__(256) void mm_step_kernel(MmParams p, int VW, int ve
     sums[1][tid >> 6] = zf;
   }
   __syncthreads();
-  const float gi = mm_log_input((sums[0][0] + sums[0][1]) + (sums[0][2] + sums[0][3]) + p.gate_b[h], p.cap);
-  const float gf = mm_log_forget((sums[1][0] + sums[1][1]) + (sums[1][2] + sums[1][3]) + p.gate_b[p.heads + h], p.cap);
-  const float next = fmaxf(gf + m, gi), keep = expf(gf + m - next), take = expf(gi - next);
+  const float gi = mm_log_gate((sums[0][0] + sums[0][1]) + (sums[0][2] + sums[0][3]) + p.gate_b[h], p.cap, p.inv_cap, false);
+  const float gf = mm_log_gate((sums[1][0] + sums[1][1]) + (sums[1][2] + sums[1][3]) + p.gate_b[p.heads + h], p.cap, p.inv_cap, true);
+  const float next = fmaxf(gf + m, gi), keep = cw_exp_quick(gf + m - next), take = cw_exp_quick(gi - next);
   const float n = keep * n_before + take * k_mine;
   if (blockIdx.z == 0) {
     if (tid < D) after[tid] = n;
@@ -602,7 +671,7 @@ __global__ __launch_bounds__(256) void mm_step_kernel(MmParams p, int VW, int ve
   for (int u = 0; u < N; ++u) red[tid * N + u] = acc[u];
   __syncthreads();
   const float total = (sums[2][0] + sums[2][1]) + (sums[2][2] + sums[2][3]);
-  const float inv = 1.0f / (fmaxf(fabsf(total), expf(-next)) + MM_EPS);
+  const float inv = __builtin_amdgcn_rcpf(fmaxf(fabsf(total), cw_exp_quick(-next)) + MM_EPS);
   for (int c = tid; c < vw; c += 256) {
     float s = 0.0f;
     for (int q = 0; q < rows_at_once; ++q) s += red[(q * cols + c / N) * N + c % N];
@@ -613,14 +682,13 @@ __global__ __launch_bounds__(256) void mm_step_kernel(MmParams p, int VW, int ve
 // ---------------------------------------------------------------- entry points
 #define MM_LDS_MOST (150 * 1024)
 static size_t mm_state_lds(int elem, int Q, int D) {
-  const int pad = elem == 2 ? 8 : 4;
-  return (size_t)Q * (mm_round(D, 16) + pad + MM_COLS + pad) * elem;
+  return (size_t)(mm_round(D, 16) + MM_COLS) * (Q + 4) * elem;
 }
 static size_t mm_out_lds(int elem, int Q, int D) {
   const int pad = elem == 2 ? 8 : 4, NK = mm_round(D, 32);
   size_t k = (size_t)Q * (NK + pad) * elem;
   if (k < (size_t)Q * (Q + 4) * 4) k = (size_t)Q * (Q + 4) * 4;
-  return (size_t)Q * (NK + pad + MM_COLS + pad) * elem + (size_t)NK * (MM_COLS + 4) * 4 + k;
+  return ((size_t)Q * (NK + pad) + (size_t)MM_COLS * (Q + 4)) * elem + (size_t)MM_COLS * (NK + 4) * 4 + k;
 }
 
 // Tokens of a chunk for keys of D elements of ``dtype`` (0: beyond the kernels).
@@ -648,7 +716,7 @@ static int mm_fill(MmParams& p, int dtype, const void* proj, int64_t stride, int
   if (q_off < 0 || k_off < 0 || v_off < 0 || q_off + heads * D > stride || k_off + heads * D > stride || v_off + heads * V > stride) return CW_ERR_ARG;
   if (state_stride < cw_matrix_memory_slot_floats(heads, D, V)) return CW_ERR_ARG;
   p.proj = proj; p.stride = stride; p.q_off = q_off; p.k_off = k_off; p.v_off = v_off; p.h = h; p.gate_w = gate_w; p.gate_b = gate_b;
-  p.width = width; p.cap = cap; p.q_scale = q_scale; p.state = state; p.state_stride = state_stride; p.n_slots = n_slots;
+  p.width = width; p.cap = cap; p.inv_cap = 1.0f / cap; p.q_scale = q_scale; p.state = state; p.state_stride = state_stride; p.n_slots = n_slots;
   p.state_slots = state_slots; p.cu_q = cu_q; p.ctx_lens = ctx_lens; p.y = y; p.heads = heads; p.D = D; p.V = V;
   p.gates = nullptr; p.items = nullptr; p.req_first = nullptr; p.added = nullptr; p.added_n = nullptr; p.chunk_f = nullptr;
   p.start_m = nullptr; p.last = nullptr; p.n_tokens = 0;

@@ -1362,7 +1362,7 @@ __global__ __launch_bounds__(256) void join_dyt_kernel(float* __restrict__ resid
     br.add(v, y, t, plane, j, H);
 #pragma unroll
     for (int u = 0; u < N; ++u) {
-      float z = tanhf(ba * v[u]) * cw_to_float(bw[j + u]);
+      float z = cw_tanh_quick(ba * v[u]) * cw_to_float(bw[j + u]);
       if (bb) z += cw_to_float(bb[j + u]);
       v[u] = r[u] + z;
     }
@@ -1372,7 +1372,7 @@ __global__ __launch_bounds__(256) void join_dyt_kernel(float* __restrict__ resid
     if (!out) continue;
 #pragma unroll
     for (int u = 0; u < N; ++u) {
-      y[u] = tanhf(a * v[u]) * cw_to_float(w[j + u]);
+      y[u] = cw_tanh_quick(a * v[u]) * cw_to_float(w[j + u]);
       if (b) y[u] += cw_to_float(b[j + u]);
     }
     if constexpr (N == 4) store4(out + i * H + j, y); else out[i * H + j] = cw_from_float<T>(y[0]);

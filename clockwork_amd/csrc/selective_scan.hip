@@ -24,7 +24,7 @@ typedef __attribute__((ext_vector_type(4))) float f32x4_t;
 typedef __attribute__((ext_vector_type(4))) unsigned int u32x4_t;
 
 #define SSC_MAX_STATE 256
-#define SSC_AHEAD 8         // tokens whose inputs a walk asks for at once
+#define SSC_AHEAD 4         // tokens whose inputs a walk asks for at once
 #define SSC_STEP_AHEAD 8    // state rows a wave of the step kernel asks for at once
 
 struct SscParams {
@@ -74,6 +74,7 @@ __global__ __launch_bounds__(256) void ssc_dt_kernel(SscParams p, int vec) {
     w[j] = (const T*)p.w_dt + (int64_t)min(c0 + j * 16 + i, p.inner - 1) * p.rank;
   }
   if constexpr (sizeof(T) == 2) {
+#pragma unroll 2
     for (int k = 0; k < p.rank; k += 32) {
       const int kk = k + kq * 8;
       union { u32x4_t u; bf16x8_t v; uint16_t s[8]; } a, b[4];
@@ -230,16 +231,17 @@ __global__ __launch_bounds__(256) void ssc_carry_kernel(SscParams p) {
   const int begin = p.req_first[r];
   int end = p.req_first[r + 1];
   while (end > begin && p.items[4 * (end - 1) + 1] >= q_len) --end;   // segments past the request's tokens (a batch of fixed shape)
-  for (int s0 = begin; s0 < end; s0 += 4) {
-    float add[4], dec[4];   // four segments' loads side by side
+  constexpr int U = 8;   // segments whose loads are on their way at once
+  for (int s0 = begin; s0 < end; s0 += U) {
+    float add[U], dec[U];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
+    for (int u = 0; u < U; ++u) {
       const int s = min(s0 + u, end - 1);
       add[u] = p.added[((int64_t)s * p.N + n) * p.inner + c];
       dec[u] = ssc_exp2(a * p.d_sum[(int64_t)s * p.inner + c]);
     }
 #pragma unroll
-    for (int u = 0; u < 4; ++u)
+    for (int u = 0; u < U; ++u)
       if (s0 + u < end) {
         p.added[((int64_t)(s0 + u) * p.N + n) * p.inner + c] = S;
         S = dec[u] * S + add[u];

@@ -31,8 +31,8 @@ CW_EXPORT int cw_short_conv(int dtype, const void* in, int64_t in_stride, int in
 // to k_plane[slot, nk], values times v_scale to v_plane[slot, nv]; a negative slot writes no cache row.
 //
 // A workgroup takes an item (a run of up to ``run`` tokens of one request). A thread convolves V channels
-// of all its tokens with the inputs in registers; queries and keys wait in LDS, float32, until the norms'
-// sums are there. The first item's workgroup alone reads the request's earlier inputs and leaves the
+// of all its tokens with the inputs in registers; the results wait in LDS, float32, until the norms' sums
+// are there. The first item's workgroup alone reads the request's earlier inputs and leaves the
 // portion's last ones, so taps - 1 <= run.
 struct QkvConv {
   const void* proj;
@@ -67,8 +67,9 @@ struct QkvConv {
 
 template <typename T, int V, int TAPS>
 __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
-  extern __shared__ __align__(16) float qkv_lds[];  // [run][nq + nk], then cosines and sines [run][2][rdims / 2]
+  extern __shared__ __align__(16) float qkv_lds[];  // [run][nq + nk + nv], then cosines and sines [run][2][rdims / 2]
   __shared__ float inv[2 * QKV_MAX_RUN];
+  __shared__ int slot_of[QKV_MAX_RUN];
   const int* item = p.items + 4 * (int64_t)blockIdx.x;
   const int req = item[0], tok0 = item[1];
   const int row0 = p.cu_q[req], q_len = p.cu_q[req + 1] - row0;
@@ -77,7 +78,10 @@ __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
   const int tid = threadIdx.x, threads = blockDim.x;
   const int QK = p.nq + p.nk, C = QK + p.nv, half = p.rdims / 2;
   const int taps = TAPS ? TAPS : p.taps;
-  float* cosines = qkv_lds + p.run * QK;
+  // what the later steps need is asked for together with the rows
+  const int t_angle = half ? min(tid / half, ntok - 1) : 0, e_angle = half ? tid % half : 0;
+  const float pos_mine = half ? (float)p.positions[row0 + tok0 + t_angle] : 0.0f, freq_mine = half ? p.freq[e_angle] : 0.0f;
+  const int slot_mine = p.slots ? p.slots[row0 + tok0 + min(tid, ntok - 1)] : -1;
   float* ring = nullptr;
   if (taps > 0) {
     const int slot = p.state_slots[req];
@@ -91,20 +95,11 @@ __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
         CwVec<T, V>::load(in + (int64_t)i * p.stride, o);
       } else {
         const int pos = pos0 + i;
+        if (pos >= 0 && ring) {
+          CwVec<float, V>::load(ring + (int64_t)(pos % taps) * C + c, o);
+        } else {
 #pragma unroll
-        for (int v = 0; v < V; ++v) o[v] = (pos >= 0 && ring) ? ring[(int64_t)(pos % taps) * C + c + v] : 0.0f;
-      }
-    };
-    auto leave = [&](int t, const float (&o)[V]) __attribute__((always_inline)) {
-      if (c < QK) {
-        CwVec<float, V>::store(qkv_lds + t * QK + c, o);
-      } else {
-        const int64_t slot = p.slots ? p.slots[row0 + tok0 + t] : -1;
-        if (slot >= 0 && slot < p.cache_rows) {
-          float y[V];
-#pragma unroll
-          for (int v = 0; v < V; ++v) y[v] = o[v] * p.v_scale;
-          CwVec<T, V>::store((T*)p.v_plane + slot * p.nv + (c - QK), y);
+          for (int v = 0; v < V; ++v) o[v] = 0.0f;
         }
       }
     };
@@ -134,9 +129,10 @@ __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
 #pragma unroll
           for (int k = 0; k < TAPS; ++k) o[v] += w[k][v] * win[k][v];
         }
-        leave(t, o);
+        CwVec<float, V>::store(qkv_lds + t * C + c, o);
       }
     } else {
+#pragma unroll 1
       for (int t = 0; t < ntok; ++t) {
         float o[V], u[V];
         if (taps == 0) {
@@ -150,10 +146,11 @@ __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
             for (int v = 0; v < V; ++v) o[v] += p.w[(int64_t)(c + v) * taps + k] * u[v];
           }
         }
-        leave(t, o);
+        CwVec<float, V>::store(qkv_lds + t * C + c, o);
       }
     }
     if (tok0 == 0 && ring) {
+#pragma unroll 1
       for (int i = max(0, q_len - (taps - 1)); i < q_len; ++i) {
         float u[V];
         CwVec<T, V>::load(in + (int64_t)i * p.stride, u);
@@ -161,10 +158,14 @@ __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
       }
     }
   }
+  if (tid < ntok) slot_of[tid] = (slot_mine >= 0 && slot_mine < p.cache_rows) ? slot_mine : -1;
+  float* cosines = qkv_lds + p.run * C;
+#pragma unroll 1
   for (int i = tid; i < ntok * half; i += threads) {
     const int t = i / half, e = i - t * half;
     float s, c;
-    sincosf((float)p.positions[row0 + tok0 + t] * p.freq[e], &s, &c);
+    if (i == tid) cw_sincos_quick(pos_mine * freq_mine, s, c);
+    else cw_sincos_quick((float)p.positions[row0 + tok0 + t] * p.freq[e], s, c);
     cosines[(2 * t) * half + e] = c * p.rot_mult;
     cosines[(2 * t + 1) * half + e] = s * p.rot_mult;
   }
@@ -174,52 +175,79 @@ __global__ __launch_bounds__(1024) void qkv_conv_store_kernel(QkvConv p) {
     // a wave a projection of a token: the sum of its squares
     for (int u = wave; u < 2 * ntok; u += waves) {
       const int t = u >> 1, n = (u & 1) ? p.nk : p.nq;
-      const float* row = qkv_lds + t * QK + ((u & 1) ? p.nq : 0);
+      const float* row = qkv_lds + t * C + ((u & 1) ? p.nq : 0);
       float ss = 0.0f;
-      for (int j = lane; j < n; j += 64) ss += row[j] * row[j];
+#pragma unroll 4
+      for (int j = lane * V; j < n; j += 64 * V) {   // V divides both sizes
+        float r[V];
+        CwVec<float, V>::load(row + j, r);
+#pragma unroll
+        for (int v = 0; v < V; ++v) ss += r[v] * r[v];
+      }
       ss = cw_wave_sum(ss);
-      if (lane == 0) inv[u] = 1.0f / sqrtf(ss / (float)n + p.eps);
+      if (lane == 0) inv[u] = rsqrtf(ss / (float)n + p.eps);
     }
     __syncthreads();
   }
-  for (int i = tid * V; i < ntok * QK; i += threads * V) {   // V divides QK
-    const int t = i / QK, c = i - t * QK;
+  // a thread keeps its channels for all tokens: their weights, and which elements turn together
+  for (int c = tid * V; c < C; c += threads * V) {
+    if (c >= QK) {
+#pragma unroll 1
+      for (int t = 0; t < ntok; ++t) {
+        if (slot_of[t] < 0) continue;
+        float o[V];
+        CwVec<float, V>::load(qkv_lds + t * C + c, o);
+#pragma unroll
+        for (int v = 0; v < V; ++v) o[v] *= p.v_scale;
+        CwVec<T, V>::store((T*)p.v_plane + (int64_t)slot_of[t] * p.nv + (c - QK), o);
+      }
+      continue;
+    }
     const bool is_q = c < p.nq;
-    const int64_t slot = p.slots ? p.slots[row0 + tok0 + t] : -1;
-    const bool stored = slot >= 0 && slot < p.cache_rows;
-    if (!is_q && !stored) continue;
-    const float* row = qkv_lds + t * QK;
-    const float* w = is_q ? p.qw : p.kw - p.nq;
-    const float iv = p.qw ? inv[2 * t + (is_q ? 0 : 1)] : 1.0f;
+    const float* w = p.qw ? (is_q ? p.qw : p.kw - p.nq) : nullptr;
     const int d = (is_q ? c : c - p.nq) % p.dim;
-    float o[V];
+    float wm[V], wp[V];
+    int pc[V];   // the partner's channel (the element's own where nothing turns)
 #pragma unroll
     for (int v = 0; v < V; ++v) {
-      float a = row[c + v] * iv;
-      if (p.qw) a *= w[c + v];
-      if (d + v < p.rdims) {
-        const bool low = d + v < half;
-        const int pc = low ? c + v + half : c + v - half, e = low ? d + v : d + v - half;
-        float b = row[pc] * iv;
-        if (p.qw) b *= w[pc];
-        const float cs = cosines[(2 * t) * half + e], sn = cosines[(2 * t + 1) * half + e];
-        a = low ? a * cs - b * sn : a * cs + b * sn;
-      }
-      o[v] = a;
+      pc[v] = d + v < p.rdims ? (d + v < half ? c + v + half : c + v - half) : c + v;
+      wm[v] = w ? w[c + v] : 1.0f;
+      wp[v] = w ? w[pc[v]] : 1.0f;
     }
-    if (is_q) CwVec<T, V>::store((T*)p.q_out + (int64_t)(row0 + tok0 + t) * p.nq + c, o);
-    else CwVec<T, V>::store((T*)p.k_plane + slot * p.nk + (c - p.nq), o);
+#pragma unroll 1
+    for (int t = 0; t < ntok; ++t) {
+      if (!is_q && slot_of[t] < 0) continue;
+      const float* row = qkv_lds + t * C;
+      const float iv = w ? inv[2 * t + (is_q ? 0 : 1)] : 1.0f;
+      float o[V];
+      CwVec<float, V>::load(row + c, o);
+#pragma unroll
+      for (int v = 0; v < V; ++v) {
+        o[v] *= iv * wm[v];
+        if (d + v < p.rdims) {
+          const bool low = d + v < half;
+          const float b = row[pc[v]] * iv * wp[v];
+          const int e = low ? d + v : d + v - half;
+          const float cs = cosines[(2 * t) * half + e], sn = cosines[(2 * t + 1) * half + e];
+          o[v] = low ? o[v] * cs - b * sn : o[v] * cs + b * sn;
+        }
+      }
+      if (is_q) CwVec<T, V>::store((T*)p.q_out + (int64_t)(row0 + tok0 + t) * p.nq + c, o);
+      else CwVec<T, V>::store((T*)p.k_plane + (int64_t)slot_of[t] * p.nk + (c - p.nq), o);
+    }
   }
 }
 
 #define QKV_LDS_MOST (150 * 1024)
-static size_t qkv_lds_bytes(int run, int qk, int rdims) { return (size_t)run * (qk + rdims) * sizeof(float); }
+static size_t qkv_lds_bytes(int run, int channels, int rdims) { return (size_t)run * (channels + rdims) * sizeof(float); }
 
 // Tokens a work item may hold (0: beyond the kernel). Few, so that a portion fills the chip; at least taps - 1.
-CW_EXPORT int cw_qkv_conv_run(int nq, int nk, int rdims, int taps) {
-  if (nq < 1 || nk < 1 || rdims < 0 || taps < 0 || taps > SHORT_CONV_MAX_TAPS) return 0;
-  int run = taps - 1 > QKV_RUN ? taps - 1 : QKV_RUN;
-  return qkv_lds_bytes(run, nq + nk, rdims) <= QKV_LDS_MOST ? run : 0;
+CW_EXPORT int cw_qkv_conv_run(int nq, int nk, int nv, int rdims, int taps) {
+  if (nq < 1 || nk < 1 || nv < 1 || rdims < 0 || taps < 0 || taps > SHORT_CONV_MAX_TAPS) return 0;
+  const int least = taps > 2 ? taps - 1 : 1;
+  for (int run = least > QKV_RUN ? least : QKV_RUN; run >= least; --run)
+    if (qkv_lds_bytes(run, nq + nk + nv, rdims) <= QKV_LDS_MOST) return run;
+  return 0;
 }
 
 CW_EXPORT int cw_qkv_conv_store(int dtype, const void* proj, int64_t stride, int off, int nq, int nk, int nv, int dim, const float* w,
@@ -228,7 +256,7 @@ CW_EXPORT int cw_qkv_conv_store(int dtype, const void* proj, int64_t stride, int
                                 float eps, const int* positions, const float* freq, int rdims, float rot_mult, float v_scale,
                                 const int* slots, void* q_out, void* k_plane, void* v_plane, int64_t cache_rows, hipStream_t stream) {
   if (!proj || !cu_q || !ctx_lens || !items || !q_out || n_items < 0 || off < 0 || nv < 1 || dim < 1) return CW_ERR_ARG;
-  const int run = cw_qkv_conv_run(nq, nk, rdims, taps);
+  const int run = cw_qkv_conv_run(nq, nk, nv, rdims, taps);
   if (!run) return CW_ERR_SIZE;
   const int64_t C = (int64_t)nq + nk + nv;
   if (off + C > stride || nq % dim || nk % dim || rdims > dim || (rdims & 1) || (rdims && (!freq || !positions))) return CW_ERR_ARG;
@@ -241,7 +269,7 @@ CW_EXPORT int cw_qkv_conv_store(int dtype, const void* proj, int64_t stride, int
   const uintptr_t align = elem * 4 - 1;
   const bool v4 = !((nq | nk | nv | dim | off) & 3) && !(stride & 3) && !(((uintptr_t)proj | (uintptr_t)q_out | (uintptr_t)k_plane | (uintptr_t)v_plane) & align) &&
                   !((uintptr_t)state & 15) && !(state_stride & 3) && !(ring_off & 3);
-  const size_t lds = qkv_lds_bytes(run, nq + nk, rdims);
+  const size_t lds = qkv_lds_bytes(run, (int)C, rdims);
   int threads = (int)((C / (v4 ? 4 : 1) + 63) / 64 * 64);
   threads = threads < 256 ? 256 : threads > 1024 ? 1024 : threads;
 #define CW_LAUNCH(T_, V_, K_)                                                                                          \

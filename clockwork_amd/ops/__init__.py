@@ -158,7 +158,7 @@ def _declare(name: str, lib: ctypes.CDLL) -> None:
             "cw_short_conv_tokens": [],
             "cw_short_conv_max_taps": [],
             "cw_short_conv": [I, P, L, I, P, L, P, P, I, P, L, L, I, P, P, P, P, I, I, I, P],
-            "cw_qkv_conv_run": [I, I, I, I],
+            "cw_qkv_conv_run": [I, I, I, I, I],
             "cw_qkv_conv_store": [I, P, L, I, I, I, I, I, P, I, P, L, L, I, P, P, P, P, I, P, P, F, P, P, I, F, F, P, P, P, P, L, P],
         },
         "selective_scan": {
@@ -2758,9 +2758,9 @@ def short_conv(x: torch.Tensor, off: int, channels: int, weight, bias, state, ri
     return out
 
 
-def qkv_conv_run(nq: int, nk: int, rot_dims: int, taps: int) -> int:
+def qkv_conv_run(nq: int, nk: int, nv: int, rot_dims: int, taps: int) -> int:
     """Tokens of one request that a work item of ``qkv_conv_store`` holds (0: beyond the kernel)."""
-    return int(_load("short_conv").cw_qkv_conv_run(nq, nk, rot_dims, taps))
+    return int(_load("short_conv").cw_qkv_conv_run(nq, nk, nv, rot_dims, taps))
 
 
 def qkv_conv_store(proj: torch.Tensor, off: int, nq: int, nk: int, nv: int, dim: int, conv, state, state_slots, cu_q, ctx_lens, items,

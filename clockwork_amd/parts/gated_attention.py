@@ -107,7 +107,7 @@ class GatedAttention(Part):
             raise NotImplementedError("a factor on what is rotated goes with a convolution or a norm over the projection")
         self.conv = params.get("conv_weight")
         if self.prepares:
-            self.conv_run = ops.qkv_conv_run(self.q_width, self.k_width, self.rot_dims, s.conv_taps)
+            self.conv_run = ops.qkv_conv_run(self.q_width, self.k_width, self.v_width, self.rot_dims, s.conv_taps)
             if not self.conv_run:
                 raise ValueError(f"projections of {self.q_width} and {self.k_width} elements with {s.conv_taps} taps are beyond the kernel")
         self.dtype = dtype
